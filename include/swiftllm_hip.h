@@ -130,9 +130,11 @@ int swl_paged_attn_decode_qkv(void *o, const float *qkv_slabs, int32_t k_splits,
 
 /* ---- Greedy sampling --------------------------------------------------------------------------
  * reference: post_layer.py:40 (`torch.argmax(logits, dim=1)`)
- * out[r] = argmax_j x[r, j] (int64), ties -> lowest j, NaNs never selected. n % 8 == 0.
+ * out[r] = argmax_j x[r, j] (int64), ties -> lowest j, NaNs never selected. n % 8 == 0. dtype may be SWL_F32.
+ * swl_logit_softcap: out fp32 = cap * tanh(x / cap). dtype may be SWL_F32.
  * scratch: swl_argmax_scratch_bytes(num_rows) bytes, 16-byte aligned. */
 size_t swl_argmax_scratch_bytes(int64_t num_rows);
+int swl_logit_softcap(float *out, const void *x, int64_t total, float cap, int32_t dtype, swl_stream_t stream);
 int swl_argmax(int64_t *out, const void *x, void *scratch, size_t scratch_bytes, int64_t num_rows, int32_t n,
                int64_t row_stride, int32_t dtype, swl_stream_t stream);
 
@@ -583,7 +585,9 @@ int swl_masked_attn_tiles(void *out, const void *q, const void *k_cache, const v
  * swl_latent_rope_store_kv: rows hold num_heads query heads [dim | rot_dim] and, at column dkv_col (< 0: none), the
  *   compressed row [kv_rank | rot_dim]. qa[t][h][kv_rank : kv_rank + rot_dim] = rotated query part; the RMS-normed latent
  *   (weight c_norm, eps) and the rotated shared key part are stored as one key head of kv_rank + rot_dim and the latent
- *   again, transposed, as one value head of kv_rank.
+ *   again, transposed, as one value head of kv_rank. half = 0: interleaved pairs, 1: dimension i turns with i + rot_dim / 2;
+ *   cosines and sines are multiplied by rot_mult. Query heads and key rows are k_dim (>= kv_rank + rot_dim) elements wide in qa
+ *   and in the pool, value rows v_dim (>= kv_rank): the columns beyond are zeroed.
  * swl_diff_head_combine: maps fp32 [T, 2, H, vdim] -> out[T, H, vdim] = unit_rms(a1 - lambda a2; eps) * mult *
  *   sigmoid(gate[t * gate_stride + h]) (gate NULL: no gate).
  * swl_head_gate: y[T, H, vdim] *= sigmoid(gate[t * gate_stride + h]) in place. */
@@ -596,7 +600,8 @@ int swl_latent_rope_store_kv(const void *proj, void *qa, const double *freq, con
                              void *v_cache, const int32_t *block_table, const int32_t *tok_seq, const int32_t *tok_pos,
                              int64_t num_tokens, int32_t num_heads, int32_t dim, int32_t rot_dim, int32_t kv_rank,
                              int64_t proj_stride, int64_t dkv_col, int64_t qa_stride, int32_t max_blocks_per_seq,
-                             int64_t block_stride, float eps, int32_t dtype, swl_stream_t stream);
+                             int64_t block_stride, float eps, int32_t half, double rot_mult, int32_t k_dim, int32_t v_dim,
+                             int32_t dtype, swl_stream_t stream);
 int swl_diff_head_combine(void *out, const float *maps, const void *gate, int64_t gate_stride, float lambda, float mult,
                           float eps, int64_t num_tokens, int32_t num_heads, int32_t vdim, int32_t dtype,
                           swl_stream_t stream);
@@ -614,8 +619,8 @@ int swl_polynorm(void *out, const void *z, float a, float b, float c, float e, f
  * dtype may be SWL_F32. */
 int swl_moe_route(int32_t *idx_out, float *w_out, const void *h, const float *router, const float *bias,
                   int64_t num_tokens, int32_t width, int32_t experts, int32_t top, int32_t dtype, swl_stream_t stream);
-int swl_moe_gate_up(void *y, const void *h, const void *gate_up, const int32_t *expert_idx, int64_t num_tokens,
-                    int32_t width, int32_t ff, int32_t top, float limit, int32_t act, int32_t dtype, swl_stream_t stream);
+int swl_moe_gate_up(void *y, const void *h, const void *gate_up, const int32_t *expert_idx, const float *in_w,
+                    int64_t num_tokens, int32_t width, int32_t ff, int32_t top, float limit, int32_t act, int32_t dtype, swl_stream_t stream);
 /* Large steps (prompt portions): assignments are sorted by expert and every expert's rows go through the library GEMM;
  * swl_glu_clamp: y[r][f] = act of [gate | up] product rows gate_up[r][2 ff]; swl_moe_combine: out[t] = sum_j w[t][j] *
  * rows[where[t * top + j]] (fp32, fixed order). dtype may be SWL_F32. */
@@ -623,13 +628,15 @@ int swl_moe_gate_up(void *y, const void *h, const void *gate_up, const int32_t *
  * multiplies it with all assignments of the expert (an expert's weights are streamed once per step). glu = 1: out = y[T * top, ff] from x = h[T, width]
  * and w = gate_up; glu = 0: out = rows[T * top, width] (plain products, for swl_moe_combine) from x = y and w = down.
  * act (swl_moe_gate_up, swl_glu_clamp): 0 the clamped unit min(g, limit) sigmoid(1.702 g) (clamp(u) + 1), 1 the plain gated
- * unit silu(g) u (limit unused); swl_moe_expert_stationary takes the latter as glu = 3. */
+ * unit silu(g) u (limit unused); swl_moe_expert_stationary takes the latter as glu = 3. in_w (NULL: none): a weight per
+ * assignment (swl_glu_clamp: per row) on the expert's input, applied to the fp32 products g and u. expert_w of the two
+ * combinations may be NULL (all one). */
 int swl_moe_expert_stationary_supported(int64_t num_tokens, int32_t width, int32_t ff, int32_t top, int32_t dtype);
-int swl_moe_expert_stationary(void *out, const void *x, const void *w, const int32_t *expert_idx, int64_t num_tokens,
-                              int32_t experts, int32_t width, int32_t ff, int32_t top, int32_t glu, float limit,
+int swl_moe_expert_stationary(void *out, const void *x, const void *w, const int32_t *expert_idx, const float *in_w,
+                              int64_t num_tokens, int32_t experts, int32_t width, int32_t ff, int32_t top, int32_t glu, float limit,
                               int32_t dtype, swl_stream_t stream);
-int swl_glu_clamp(void *y, const void *gate_up, int64_t num_rows, int32_t ff, float limit, int32_t act, int32_t dtype,
-                  swl_stream_t stream);
+int swl_glu_clamp(void *y, const void *gate_up, const float *in_w, int64_t num_rows, int32_t ff, float limit, int32_t act,
+                  int32_t dtype, swl_stream_t stream);
 int swl_moe_combine(void *out, const void *rows, const int64_t *where, const float *expert_w, int64_t num_tokens,
                     int32_t width, int32_t top, int32_t dtype, swl_stream_t stream);
 int swl_moe_down_combine(void *out, const void *y, const void *down, const int32_t *expert_idx, const float *expert_w,
@@ -693,10 +700,10 @@ int swl_gated_head_rmsnorm(void *out, const float *o, const void *gate, int64_t 
  * s = sigmoid(router[experts, width] h) in fp32. Experts are chosen by s + correction (NULL: by s): the experts form
  * group_count equal groups of neighbours, a group's score is the sum of its two largest choice scores, only experts of the
  * group_keep best groups are eligible (group_keep = group_count: all), of these the `top` largest. w_out = the chosen
- * experts' s divided by their sum (+ 1e-20). dtype may be SWL_F32. */
+ * experts' s, divided by their sum (+ 1e-20) when normalize is set. dtype may be SWL_F32. */
 int swl_moe_route_grouped(int32_t *idx_out, float *w_out, const void *h, const float *router, const float *correction,
                           int64_t num_tokens, int32_t width, int32_t experts, int32_t top, int32_t group_count,
-                          int32_t group_keep, int32_t dtype, swl_stream_t stream);
+                          int32_t group_keep, int32_t normalize, int32_t dtype, swl_stream_t stream);
 
 /* ---- projections with biases: per-head q/k RMS norm + value blend + KV store (pool layout of swl_qknorm_store_kv) -----------
  * q_h <- (q_h + q_b) / rms * q_w (in place; q_w[dim] shared by the heads, NULL: no weight), keys likewise into the pool,
@@ -753,6 +760,50 @@ int swl_gated_group_rmsnorm(void *out, const float *y, const void *gate, int64_t
  * out (may be NULL) = x in the compute dtype, or x / rms(x) * w2 when w2 is given. dtype may be SWL_F32. */
 int swl_post_norm_add(float *x, const void *a, const float *wa, const void *b, const float *wb, float coef, const float *w1,
                       void *out, const float *w2, float eps, int64_t num_rows, int32_t width, int32_t dtype,
+                      swl_stream_t stream);
+
+/* ---- attention projections with biases, q/k norm, rotary and keys as values (csrc/rope_kv.hip) -----------------------------------
+ * rows [q: num_q_heads of dim | k: num_k_heads of dim | v: num_v_heads of vdim]. Per query / key head: + bias (fp32, NULL: none),
+ * RMS norm over dim with a weight shared by the heads (NULL: no norm), rotation of the first rot_dims dimensions (half = 0:
+ * interleaved pairs, 1: dimension i with i + rot_dims / 2; cosines and sines times rot_mult). q, times q_mult[head] (NULL: 1), goes
+ * to q_out (heads k_dim wide), k to the K pool (rows k_dim wide), and to the V pool (v_dim wide): the value columns, or with
+ * keys_as_values (num_v_heads = 0, vdim = dim) the keys after the bias only. Columns beyond dim / vdim are zeroed. k_cache NULL:
+ * queries only. dtype may be SWL_F32. */
+int swl_qk_norm_rope_store_kv(const void *rows, void *q_out, const float *q_b, const float *k_b, const float *q_w,
+                              const float *k_w, const float *q_mult, const double *freq, void *k_cache, void *v_cache,
+                              const int32_t *block_table, const int32_t *tok_seq, const int32_t *tok_pos, int64_t num_tokens,
+                              int32_t num_q_heads, int32_t num_k_heads, int32_t num_v_heads, int32_t dim, int32_t vdim,
+                              int32_t rot_dims, int32_t half, double rot_mult, int64_t tok_stride, int64_t q_out_stride,
+                              int32_t k_dim, int32_t v_dim, int32_t keys_as_values, int32_t max_blocks_per_seq,
+                              int64_t block_stride, float eps, int32_t dtype, swl_stream_t stream);
+
+/* ---- fp32 residual of several streams, hyper-connections (csrc/hyper_stream.hip) ------------------------------------------------
+ * x [rows, streams, width] fp32. swl_embed_streams: every stream = embed[token]. swl_hyper_step: with y (+ y2, + y_bias[width])
+ * the previous sublayer's result, X_t <- sum_s mix[s][t] X_s + outw[t] y (all from the old streams); then, with h given,
+ * u = sum_s inw[s] X_s (inw NULL: plain sum) and h = u / rms(u in `groups` equal parts; eps) * norm_w. y NULL: norm only, of
+ * rows row_idx when given; h NULL: update only. At most 8 streams. dtype (y, y2, h) may be SWL_F32. */
+int swl_embed_streams(float *x, const void *embed, const int32_t *tokens, int64_t num_tokens, int32_t width, int32_t streams,
+                      int32_t dtype, swl_stream_t stream);
+int swl_hyper_step(float *x, const void *y, const void *y2, const float *y_bias, const float *mix, const float *outw,
+                   const float *inw, const float *norm_w, void *h, const int32_t *row_idx, int64_t num_rows, int32_t width,
+                   int32_t streams, int32_t groups, float eps, int32_t dtype, swl_stream_t stream);
+
+/* ---- minGRU (csrc/min_gru.hip) -----------------------------------------------------------------------------------------------------
+ * proj rows [z | u | gate] of width columns each; per channel a = sigmoid(z + z_b), c = u' + 1/2 (u' = u + u_b >= 0) or sigmoid(u'),
+ * S <- (1 - a) S + a c in fp32 (the state: width floats at s_off inside the sequence's slot), out = S * silu(gate).
+ * swl_min_gru_apply alone serves steps in which every portion is ONE chunk (chunk_row0, chunk_cnt: runs of consecutive tokens
+ * of one sequence; start NULL). Otherwise swl_min_gru_chunks composes every chunk into part [chunks, 2, width],
+ * swl_min_gru_carry walks a portion's chunks of chunk_tokens tokens (from seq_chunk0 on), updates the slots and leaves the
+ * chunks' start states in part[:, 0], and swl_min_gru_apply takes them as `start`. dtype may be SWL_F32. */
+int swl_min_gru_chunks(float *part, const void *proj, int64_t proj_stride, const float *z_b, const float *u_b,
+                       const int32_t *chunk_row0, const int32_t *chunk_cnt, int32_t num_chunks, int32_t width, int32_t dtype,
+                       swl_stream_t stream);
+int swl_min_gru_carry(float *part, float *state, int64_t slot_stride, int64_t s_off, const int32_t *seq_row0,
+                      const int32_t *seq_cnt, const int32_t *seq_chunk0, const int32_t *tok_pos, const int32_t *tok_state,
+                      int32_t num_seqs, int32_t chunk_tokens, int32_t width, swl_stream_t stream);
+int swl_min_gru_apply(void *out, const void *proj, int64_t proj_stride, const float *z_b, const float *u_b, const float *start,
+                      float *state, int64_t slot_stride, int64_t s_off, const int32_t *chunk_row0, const int32_t *chunk_cnt,
+                      const int32_t *tok_pos, const int32_t *tok_state, int32_t num_chunks, int32_t width, int32_t dtype,
                       swl_stream_t stream);
 
 #ifdef __cplusplus

@@ -27,6 +27,7 @@ _P = ctypes.c_void_p
 _I32 = ctypes.c_int32
 _I64 = ctypes.c_int64
 _F32 = ctypes.c_float
+_F64 = ctypes.c_double
 
 # name -> argument ctypes, in the order of include/swiftllm_hip.h. tests/test_abi.py checks this table
 # against the header (symbol set and arity) and against the built library's exports.
@@ -108,14 +109,14 @@ SIGNATURES = {
                               _F32, _I32, _I64, _I32, _P, _I64, _I32, _P, _I32, _I32, _I32, _I32, _P],
     "swl_rope_store_kv": [_P, _P, _P, _P, _P, _P, _P, _I64, _I32, _I32, _I32, _I32, _I32, _I32, _I64, _I32, _I64, _I32, _P],
     "swl_latent_rope_store_kv": [_P, _P, _P, _P, _P, _P, _P, _P, _P, _I64, _I32, _I32, _I32, _I32, _I64, _I64, _I64, _I32,
-                                 _I64, _F32, _I32, _P],
+                                 _I64, _F32, _I32, _F64, _I32, _I32, _I32, _P],
     "swl_diff_head_combine": [_P, _P, _P, _I64, _F32, _F32, _F32, _I64, _I32, _I32, _I32, _P],
     "swl_head_gate": [_P, _P, _I64, _I64, _I32, _I32, _I32, _P],
     "swl_polynorm": [_P, _P, _F32, _F32, _F32, _F32, _F32, _I64, _I32, _I32, _P],
     "swl_moe_route": [_P, _P, _P, _P, _P, _I64, _I32, _I32, _I32, _I32, _P],
-    "swl_moe_gate_up": [_P, _P, _P, _P, _I64, _I32, _I32, _I32, _F32, _I32, _I32, _P],
-    "swl_moe_expert_stationary": [_P, _P, _P, _P, _I64, _I32, _I32, _I32, _I32, _I32, _F32, _I32, _P],
-    "swl_glu_clamp": [_P, _P, _I64, _I32, _F32, _I32, _I32, _P],
+    "swl_moe_gate_up": [_P, _P, _P, _P, _P, _I64, _I32, _I32, _I32, _F32, _I32, _I32, _P],
+    "swl_moe_expert_stationary": [_P, _P, _P, _P, _P, _I64, _I32, _I32, _I32, _I32, _I32, _F32, _I32, _P],
+    "swl_glu_clamp": [_P, _P, _P, _I64, _I32, _F32, _I32, _I32, _P],
     "swl_moe_combine": [_P, _P, _P, _P, _I64, _I32, _I32, _I32, _P],
     "swl_moe_down_combine": [_P, _P, _P, _P, _P, _I64, _I32, _I32, _I32, _I32, _P],
     "swl_moe_route_scores": [_P, _P, _P, _P, _P, _I64, _I32, _I32, _I32, _F32, _I32, _P],
@@ -129,7 +130,7 @@ SIGNATURES = {
                        _I32, _I32, _I32, _P],
     "swl_delta_rule": [_P, _P, _P, _P, _P, _P, _P, _P, _I64, _I64, _P, _P, _P, _P, _I32, _I32, _I32, _I32, _I32, _P],
     "swl_gated_head_rmsnorm": [_P, _P, _P, _I64, _P, _F32, _I64, _I32, _I32, _I32, _P],
-    "swl_moe_route_grouped": [_P, _P, _P, _P, _P, _I64, _I32, _I32, _I32, _I32, _I32, _I32, _P],
+    "swl_moe_route_grouped": [_P, _P, _P, _P, _P, _I64, _I32, _I32, _I32, _I32, _I32, _I32, _I32, _P],
     "swl_qkv_bias_norm_store": [_P, _P, _P, _P, _P, _P, _P, _I64, _F32, _P, _P, _P, _P, _P, _I64, _I32, _I32, _I32, _I32,
                                 _I64, _I32, _I64, _F32, _I32, _P],
     "swl_sigmoid_attn": [_P, _P, _P, _P, _P, _P, _P, _P, _P, _P, _P, _I64, _I32, _I32, _I32, _I32, _I64, _I32, _F32, _I32,
@@ -140,6 +141,14 @@ SIGNATURES = {
                      _I32, _I32, _P],
     "swl_ssd_scan": [_P, _P, _P, _P, _P, _P, _I64, _I64, _P, _P, _P, _P, _I32, _I32, _I32, _I32, _I32, _P],
     "swl_gated_group_rmsnorm": [_P, _P, _P, _I64, _P, _F32, _I64, _I32, _I32, _I32, _P],
+    "swl_logit_softcap": [_P, _P, _I64, _F32, _I32, _P],
+    "swl_qk_norm_rope_store_kv": [_P, _P, _P, _P, _P, _P, _P, _P, _P, _P, _P, _P, _P, _I64, _I32, _I32, _I32, _I32, _I32, _I32,
+                                  _I32, _F64, _I64, _I64, _I32, _I32, _I32, _I32, _I64, _F32, _I32, _P],
+    "swl_embed_streams": [_P, _P, _P, _I64, _I32, _I32, _I32, _P],
+    "swl_hyper_step": [_P, _P, _P, _P, _P, _P, _P, _P, _P, _P, _I64, _I32, _I32, _I32, _F32, _I32, _P],
+    "swl_min_gru_chunks": [_P, _P, _I64, _P, _P, _P, _P, _I32, _I32, _I32, _P],
+    "swl_min_gru_carry": [_P, _P, _I64, _I64, _P, _P, _P, _P, _P, _I32, _I32, _I32, _P],
+    "swl_min_gru_apply": [_P, _P, _I64, _P, _P, _P, _P, _I64, _I64, _P, _P, _P, _P, _I32, _I32, _I32, _P],
     "swl_post_norm_add": [_P, _P, _P, _P, _P, _F32, _P, _P, _P, _F32, _I64, _I32, _I32, _P],
 }
 # Entry points that do not follow the "int rc = f(...)" convention.

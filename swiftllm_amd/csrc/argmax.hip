@@ -6,6 +6,9 @@
 // workgroup scans its slice with 16-byte loads and leaves one (value, index) candidate; the second
 // kernel picks among the candidates. Comparison is on the stored values (exact, no rounding), NaNs are
 // never selected (torch would return the first NaN — logits of a healthy model have none).
+//
+//   swl_logit_softcap: out = cap * tanh(x / cap) in fp32 (the capped values crowd below cap: a 16-bit result would make ties of
+//   logits that differ); the argmax also takes fp32 rows.
 #include "swl_common.h"
 
 namespace swl {
@@ -61,6 +64,12 @@ __global__ __launch_bounds__(256) void argmax_partial_kernel(const T *__restrict
     }
 }
 
+template <typename T>
+__global__ __launch_bounds__(256) void logit_softcap_kernel(float *out, const T *x, int64_t total, float cap) {
+    const int64_t i = static_cast<int64_t>(blockIdx.x) * 256 + threadIdx.x;
+    if (i < total) out[i] = cap * tanhf(to_f(x[i]) / cap);
+}
+
 __global__ __launch_bounds__(64) void argmax_final_kernel(const float *__restrict__ part_val,
                                                           const int *__restrict__ part_idx,
                                                           int64_t *__restrict__ out) {
@@ -91,11 +100,24 @@ extern "C" int swl_argmax(int64_t *out, const void *x, void *scratch, size_t scr
     float *pv = static_cast<float *>(scratch);
     int *pi = reinterpret_cast<int *>(pv + num_rows * swl::kArgmaxSplits);
     hipStream_t s = static_cast<hipStream_t>(stream);
-    SWL_DISPATCH_DTYPE(dtype, T, {
+    SWL_DISPATCH_DTYPE3(dtype, T, {
         hipLaunchKernelGGL((swl::argmax_partial_kernel<T>), dim3(swl::kArgmaxSplits, static_cast<unsigned>(num_rows)),
                            dim3(256), 0, s, static_cast<const T *>(x), row_stride, n, pv, pi);
         hipLaunchKernelGGL(swl::argmax_final_kernel, dim3(static_cast<unsigned>(num_rows)), dim3(64), 0, s, pv, pi,
                            out);
+    });
+    return swl::check_launch();
+}
+
+extern "C" int swl_logit_softcap(float *out, const void *x, int64_t total, float cap, int32_t dtype, swl_stream_t stream) {
+    if (total < 0 || !(cap > 0.f)) return SWL_ERR_BAD_ARG;
+    if (total == 0) return SWL_OK;
+    if (!out || !x) return SWL_ERR_BAD_ARG;
+    const int64_t blocks = (total + 255) / 256;
+    if (blocks > 0x7fffffffLL) return SWL_ERR_UNSUPPORTED;
+    SWL_DISPATCH_DTYPE3(dtype, T, {
+        hipLaunchKernelGGL((swl::logit_softcap_kernel<T>), dim3(static_cast<unsigned>(blocks)), dim3(256), 0,
+                           static_cast<hipStream_t>(stream), out, static_cast<const T *>(x), total, cap);
     });
     return swl::check_launch();
 }

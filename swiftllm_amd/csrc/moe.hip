@@ -10,7 +10,10 @@
 //
 //   swl_moe_route_grouped: scores s = sigmoid(router h); experts are CHOSEN by s + correction, inside the `keep` best of
 //                         `count` equal groups of neighbouring experts (a group's score: the sum of its two largest choice
-//                         scores); the weights are the chosen experts' s divided by their sum.
+//                         scores); the weights are the chosen experts' s, divided by their sum when `normalize` is set.
+//   in_w (swl_moe_gate_up, swl_glu_clamp, swl_moe_expert_stationary): a weight per assignment on the expert's INPUT. The first
+//                         products are linear, so it multiplies their fp32 sums: act(w g, w u). The combination then takes no
+//                         weights (NULL: all one).
 //   act (swl_moe_gate_up, swl_glu_clamp; glu = 3 of swl_moe_expert_stationary): 0 the clamped unit above, 1 the plain gated
 //                         unit y = silu(g) * u.
 //
@@ -139,7 +142,7 @@ template <typename T>
 __global__ __launch_bounds__(kMoeThreads) void moe_route_grouped_kernel(int32_t *idx_out, float *w_out, const T *h,
                                                                         const float *router, const float *correction,
                                                                         int width, int experts, int top, int count,
-                                                                        int keep) {
+                                                                        int keep, int normalize) {
     extern __shared__ float lds[];
     float *hf = lds;                    // [width]
     float *score = hf + width;          // [experts] s = sigmoid(logit)
@@ -236,7 +239,7 @@ __global__ __launch_bounds__(kMoeThreads) void moe_route_grouped_kernel(int32_t 
         __threadfence_block();
     }
     if (lane == 0) {
-        const float mult = 1.0f / (denom + 1e-20f);
+        const float mult = normalize ? 1.0f / (denom + 1e-20f) : 1.0f;
         for (int j = 0; j < top; ++j) w_out[t * top + j] *= mult;
     }
 }
@@ -244,8 +247,8 @@ __global__ __launch_bounds__(kMoeThreads) void moe_route_grouped_kernel(int32_t 
 // grid (assignments, ceil(ff / 64)): wave w of the workgroup computes ff rows f0 + w, f0 + w + 4, ...
 template <typename T>
 __global__ __launch_bounds__(kMoeThreads) void moe_gate_up_kernel(T *y, const T *h, const T *gate_up,
-                                                                  const int32_t *expert_idx, int width, int ff, int top,
-                                                                  float limit, int act) {
+                                                                  const int32_t *expert_idx, const float *in_w, int width,
+                                                                  int ff, int top, float limit, int act) {
     extern __shared__ float lds[];
     float *hf = lds;    // [width]
     const int64_t a = blockIdx.x;           // assignment = token * top + j
@@ -262,6 +265,10 @@ __global__ __launch_bounds__(kMoeThreads) void moe_gate_up_kernel(T *y, const T 
         float g = lane_dot(hf, rg, width, lane), u = lane_dot(hf, ru, width, lane);
         g = wave_allreduce_sum(g);
         u = wave_allreduce_sum(u);
+        if (in_w) {
+            g *= in_w[a];
+            u *= in_w[a];
+        }
         if (lane == 0) y[a * ff + f] = to_t<T>(gated_unit(g, u, limit, act));
     }
 }
@@ -332,7 +339,7 @@ __global__ __launch_bounds__(kMoeThreads) void moe_down_combine_kernel(T *out, c
             const T *wr = down + (static_cast<int64_t>(e) * width + c) * ff;
             const T *yr = y + (t * top + j) * ff;
             float a = wave_allreduce_sum(lane_dot2(yr, wr, ff, lane));
-            total += expert_w[t * top + j] * a;
+            total += expert_w ? expert_w[t * top + j] * a : a;
         }
         if (lane == 0) out[t * width + c] = to_t<T>(total);
     }
@@ -353,8 +360,8 @@ constexpr int kEsMaxAssign = 1024;  // assignments per step (the sorted library 
 
 template <typename T, int MODE>
 __global__ __launch_bounds__(kMoeThreads, 2) void moe_expert_stationary_kernel(T *out, const T *x, const T *w,
-                                                                            const int32_t *expert_idx, int assignments,
-                                                                            int K, int N, int top, float limit, int ksplit) {
+                                                                            const int32_t *expert_idx, const float *in_w,
+                                                                            int assignments, int K, int N, int top, float limit, int ksplit) {
     // ksplit = 1: every wave of the workgroup owns 16 outputs and the whole reduction. ksplit = waves of the workgroup: all
     // waves own the SAME 16 outputs and a quarter (half) of the reduction each; their accumulators meet in LDS and wave 0
     // finishes (short reductions and few outputs would otherwise leave most of the chip idle in a decode step).
@@ -474,7 +481,10 @@ __global__ __launch_bounds__(kMoeThreads, 2) void moe_expert_stationary_kernel(T
                     const int n = n0 + 4 * lq + r;
                     if (n < N) {
                         float v = accg[t][r];
-                        if constexpr (GLU) v = gated_unit(v, accu[t][r], limit, MODE == 3 ? 1 : 0);
+                        if constexpr (GLU) {
+                            const float iw = in_w ? in_w[arow[t]] : 1.f;
+                            v = gated_unit(v * iw, accu[t][r] * iw, limit, MODE == 3 ? 1 : 0);
+                        }
                         if constexpr (MODE == 2) {
                             v = fmaxf(v, 0.f);
                             v *= v;
@@ -487,15 +497,33 @@ __global__ __launch_bounds__(kMoeThreads, 2) void moe_expert_stationary_kernel(T
     }
 }
 
-// y[r][f] = act(gu[r][f], gu[r][ff + f]) for rows of [gate | up] products that came from a library GEMM
+// y[r][f] = act(w[r] gu[r][f], w[r] gu[r][ff + f]) for rows of [gate | up] products that came from a library GEMM (in_w NULL: 1)
 template <typename T>
-__global__ __launch_bounds__(kMoeThreads) void glu_clamp_kernel(T *y, const T *gu, int64_t total, int ff, float limit,
-                                                                int act) {
+__global__ __launch_bounds__(kMoeThreads) void glu_clamp_kernel(T *y, const T *gu, const float *in_w, int64_t total, int ff,
+                                                                float limit, int act) {
     const int64_t i = static_cast<int64_t>(blockIdx.x) * kMoeThreads + threadIdx.x;
     if (i >= total) return;
     const int64_t r = i / ff;
     const int f = static_cast<int>(i - r * ff);
-    y[i] = to_t<T>(gated_unit(to_f(gu[r * 2 * ff + f]), to_f(gu[r * 2 * ff + ff + f]), limit, act));
+    const float w = in_w ? in_w[r] : 1.f;
+    y[i] = to_t<T>(gated_unit(w * to_f(gu[r * 2 * ff + f]), w * to_f(gu[r * 2 * ff + ff + f]), limit, act));
+}
+
+// the same for 16-bit rows of a multiple of 8 elements on 16-byte boundaries: 8 elements (16 bytes) per lane
+template <typename T>
+__global__ __launch_bounds__(kMoeThreads) void glu_clamp_wide_kernel(T *y, const T *gu, const float *in_w, int64_t total8,
+                                                                     int ff8, float limit, int act) {
+    const int64_t i = static_cast<int64_t>(blockIdx.x) * kMoeThreads + threadIdx.x;
+    if (i >= total8) return;
+    const int64_t r = i / ff8;
+    const int f = static_cast<int>(i - r * ff8) * 8;
+    const int64_t ff = static_cast<int64_t>(ff8) * 8;
+    const float w = in_w ? in_w[r] : 1.f;
+    const vec8_t<T> g = load8(gu + r * 2 * ff + f), u = load8(gu + r * 2 * ff + ff + f);
+    vec8_t<T> o;
+#pragma unroll
+    for (int j = 0; j < 8; ++j) o[j] = to_t<T>(gated_unit(w * to_f(g[j]), w * to_f(u[j]), limit, act));
+    store8(y + r * ff + f, o);
 }
 
 // out[t] = sum_j w[t][j] * rows[where[t * top + j]]  (fp32 sum in the order j = 0, 1, ...)
@@ -505,7 +533,7 @@ __global__ __launch_bounds__(kMoeThreads) void moe_combine_kernel(T *out, const 
     const int64_t t = blockIdx.x;
     for (int c = threadIdx.x; c < width; c += kMoeThreads) {
         float a = 0.f;
-        for (int j = 0; j < top; ++j) a += w[t * top + j] * to_f(rows[where[t * top + j] * width + c]);
+        for (int j = 0; j < top; ++j) a += (w ? w[t * top + j] : 1.f) * to_f(rows[where[t * top + j] * width + c]);
         out[t * width + c] = to_t<T>(a);
     }
 }
@@ -520,7 +548,7 @@ extern "C" int swl_moe_expert_stationary_supported(int64_t num_tokens, int32_t w
     return num_tokens * top <= swl::kEsMaxAssign;
 }
 
-extern "C" int swl_moe_expert_stationary(void *out, const void *x, const void *w, const int32_t *expert_idx,
+extern "C" int swl_moe_expert_stationary(void *out, const void *x, const void *w, const int32_t *expert_idx, const float *in_w,
                                          int64_t num_tokens, int32_t experts, int32_t width, int32_t ff, int32_t top,
                                          int32_t glu, float limit, int32_t dtype, swl_stream_t stream) {
     if (num_tokens < 0 || experts <= 0 || top <= 0) return SWL_ERR_BAD_ARG;
@@ -543,34 +571,43 @@ extern "C" int swl_moe_expert_stationary(void *out, const void *x, const void *w
         if (glu == 1)
             hipLaunchKernelGGL((swl::moe_expert_stationary_kernel<T, 1>), grid, dim3(64 * nw), lds, s,
                                static_cast<T *>(out), static_cast<const T *>(x), static_cast<const T *>(w), expert_idx,
-                               assignments, K, N, top, limit, ksplit);
+                               in_w, assignments, K, N, top, limit, ksplit);
         else if (glu == 2)
             hipLaunchKernelGGL((swl::moe_expert_stationary_kernel<T, 2>), grid, dim3(64 * nw), lds, s,
                                static_cast<T *>(out), static_cast<const T *>(x), static_cast<const T *>(w), expert_idx,
-                               assignments, K, N, top, limit, ksplit);
+                               in_w, assignments, K, N, top, limit, ksplit);
         else if (glu == 3)
             hipLaunchKernelGGL((swl::moe_expert_stationary_kernel<T, 3>), grid, dim3(64 * nw), lds, s,
                                static_cast<T *>(out), static_cast<const T *>(x), static_cast<const T *>(w), expert_idx,
-                               assignments, K, N, top, limit, ksplit);
+                               in_w, assignments, K, N, top, limit, ksplit);
         else
             hipLaunchKernelGGL((swl::moe_expert_stationary_kernel<T, 0>), grid, dim3(64 * nw), lds, s,
                                static_cast<T *>(out), static_cast<const T *>(x), static_cast<const T *>(w), expert_idx,
-                               assignments, K, N, top, limit, ksplit);
+                               in_w, assignments, K, N, top, limit, ksplit);
     });
     return swl::check_launch();
 }
 
-extern "C" int swl_glu_clamp(void *y, const void *gate_up, int64_t num_rows, int32_t ff, float limit, int32_t act,
-                             int32_t dtype, swl_stream_t stream) {
+extern "C" int swl_glu_clamp(void *y, const void *gate_up, const float *in_w, int64_t num_rows, int32_t ff, float limit,
+                             int32_t act, int32_t dtype, swl_stream_t stream) {
     if (num_rows < 0 || ff <= 0 || act < 0 || act > 1) return SWL_ERR_BAD_ARG;
     if (num_rows == 0) return SWL_OK;
     if (!y || !gate_up) return SWL_ERR_BAD_ARG;
-    const int64_t total = num_rows * ff;
+    const bool wide = dtype != SWL_F32 && ff % 8 == 0 && swl::aligned16(y) && swl::aligned16(gate_up);
+    const int64_t total = num_rows * ff / (wide ? 8 : 1);
     const int64_t blocks = (total + swl::kMoeThreads - 1) / swl::kMoeThreads;
     if (blocks > 0x7fffffffLL) return SWL_ERR_UNSUPPORTED;
+    if (wide) {
+        SWL_DISPATCH_DTYPE(dtype, T, {
+            hipLaunchKernelGGL((swl::glu_clamp_wide_kernel<T>), dim3(static_cast<unsigned>(blocks)), dim3(swl::kMoeThreads), 0,
+                               static_cast<hipStream_t>(stream), static_cast<T *>(y), static_cast<const T *>(gate_up), in_w,
+                               total, ff / 8, limit, act);
+        });
+        return swl::check_launch();
+    }
     SWL_DISPATCH_DTYPE3(dtype, T, {
         hipLaunchKernelGGL((swl::glu_clamp_kernel<T>), dim3(static_cast<unsigned>(blocks)), dim3(swl::kMoeThreads), 0,
-                           static_cast<hipStream_t>(stream), static_cast<T *>(y), static_cast<const T *>(gate_up), total,
+                           static_cast<hipStream_t>(stream), static_cast<T *>(y), static_cast<const T *>(gate_up), in_w, total,
                            ff, limit, act);
     });
     return swl::check_launch();
@@ -580,7 +617,7 @@ extern "C" int swl_moe_combine(void *out, const void *rows, const int64_t *where
                                int64_t num_tokens, int32_t width, int32_t top, int32_t dtype, swl_stream_t stream) {
     if (num_tokens < 0 || width <= 0 || top <= 0) return SWL_ERR_BAD_ARG;
     if (num_tokens == 0) return SWL_OK;
-    if (!out || !rows || !where || !expert_w) return SWL_ERR_BAD_ARG;
+    if (!out || !rows || !where) return SWL_ERR_BAD_ARG;
     if (num_tokens > 0x7fffffffLL) return SWL_ERR_UNSUPPORTED;
     SWL_DISPATCH_DTYPE3(dtype, T, {
         hipLaunchKernelGGL((swl::moe_combine_kernel<T>), dim3(static_cast<unsigned>(num_tokens)), dim3(swl::kMoeThreads), 0,
@@ -622,7 +659,7 @@ extern "C" int swl_moe_route_scores(int32_t *idx_out, float *w_out, const void *
     return swl::check_launch();
 }
 
-extern "C" int swl_moe_gate_up(void *y, const void *h, const void *gate_up, const int32_t *expert_idx,
+extern "C" int swl_moe_gate_up(void *y, const void *h, const void *gate_up, const int32_t *expert_idx, const float *in_w,
                                int64_t num_tokens, int32_t width, int32_t ff, int32_t top, float limit, int32_t act,
                                int32_t dtype, swl_stream_t stream) {
     if (num_tokens < 0 || width <= 0 || ff <= 0 || top <= 0 || act < 0 || act > 1) return SWL_ERR_BAD_ARG;
@@ -635,7 +672,7 @@ extern "C" int swl_moe_gate_up(void *y, const void *h, const void *gate_up, cons
     SWL_DISPATCH_DTYPE3(dtype, T, {
         hipLaunchKernelGGL((swl::moe_gate_up_kernel<T>), grid, dim3(swl::kMoeThreads), lds,
                            static_cast<hipStream_t>(stream), static_cast<T *>(y), static_cast<const T *>(h),
-                           static_cast<const T *>(gate_up), expert_idx, width, ff, top, limit, act);
+                           static_cast<const T *>(gate_up), expert_idx, in_w, width, ff, top, limit, act);
     });
     return swl::check_launch();
 }
@@ -645,7 +682,7 @@ extern "C" int swl_moe_down_combine(void *out, const void *y, const void *down, 
                                     int32_t dtype, swl_stream_t stream) {
     if (num_tokens < 0 || width <= 0 || ff <= 0 || top <= 0) return SWL_ERR_BAD_ARG;
     if (num_tokens == 0) return SWL_OK;
-    if (!out || !y || !down || !expert_idx || !expert_w) return SWL_ERR_BAD_ARG;
+    if (!out || !y || !down || !expert_idx) return SWL_ERR_BAD_ARG;
     if (num_tokens > 0x7fffffffLL || (width + 63) / 64 > 65535) return SWL_ERR_UNSUPPORTED;
     const dim3 grid(static_cast<unsigned>(num_tokens), static_cast<unsigned>((width + 63) / 64));
     SWL_DISPATCH_DTYPE3(dtype, T, {
@@ -700,7 +737,8 @@ extern "C" int swl_relu_sq(void *y, const void *z, int64_t num_rows, int32_t ff,
 
 extern "C" int swl_moe_route_grouped(int32_t *idx_out, float *w_out, const void *h, const float *router,
                                      const float *correction, int64_t num_tokens, int32_t width, int32_t experts, int32_t top,
-                                     int32_t group_count, int32_t group_keep, int32_t dtype, swl_stream_t stream) {
+                                     int32_t group_count, int32_t group_keep, int32_t normalize, int32_t dtype,
+                                     swl_stream_t stream) {
     if (num_tokens < 0 || width <= 0 || experts <= 0 || top <= 0 || top > experts) return SWL_ERR_BAD_ARG;
     if (group_count < 1 || group_keep < 1 || group_keep > group_count || experts % group_count) return SWL_ERR_BAD_ARG;
     if (static_cast<int64_t>(group_keep) * (experts / group_count) < top) return SWL_ERR_BAD_ARG;
@@ -711,7 +749,8 @@ extern "C" int swl_moe_route_grouped(int32_t *idx_out, float *w_out, const void 
     SWL_DISPATCH_DTYPE3(dtype, T, {
         hipLaunchKernelGGL((swl::moe_route_grouped_kernel<T>), dim3(static_cast<unsigned>(num_tokens)),
                            dim3(swl::kMoeThreads), lds, static_cast<hipStream_t>(stream), idx_out, w_out,
-                           static_cast<const T *>(h), router, correction, width, experts, top, group_count, group_keep);
+                           static_cast<const T *>(h), router, correction, width, experts, top, group_count, group_keep,
+                           normalize);
     });
     return swl::check_launch();
 }

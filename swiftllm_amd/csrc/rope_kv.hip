@@ -1,14 +1,18 @@
-// rope_kv.hip — rotary positions on interleaved pairs fused with the paged KV store, and what attention heads need after the
-// softmax when they are gated or combined.
+// rope_kv.hip — rotary positions fused with the paged KV store, and what attention heads need after the softmax when they are
+// gated or combined.
 //
-// Rotation: inside a head, dimension 2i is paired with dimension 2i + 1 for i < rot_dims / 2; the pair (u, v) of a token at
-// position p becomes (u cos a - v sin a, v cos a + u sin a), a = p * freq[i]. The frequencies come from the host as a
-// float64 table (base^(-2i / rot_dims), evaluated once per model); the angle and its sine and cosine are evaluated in
-// float64 per (token, i) into LDS and used in fp32 by every head of the token — exact to fp32 rounding at any position.
-// Dimensions from rot_dims on pass unchanged.
+// Rotation: inside a head, for i < rot_dims / 2, dimension 2i is paired with dimension 2i + 1 (interleaved pairs) or dimension i
+// with dimension i + rot_dims / 2 (halves: the kernels that take `half`); the pair (u, v) of a token at position p becomes
+// (u cos a - v sin a, v cos a + u sin a), a = p * freq[i]. The frequencies come from the host as a float64 table (evaluated once
+// per model, any interpolation included); the angle and its sine and cosine are evaluated in float64 per (token, i) into LDS —
+// times a constant, where the kernel takes one — and used in fp32 by every head of the token: exact to fp32 rounding at any
+// position. Dimensions from rot_dims on pass unchanged.
 //
 //   swl_rope_store_kv         rows [q: nq heads of d | k: nk heads of d | v: nv heads of dv]: q rotated in place, k rotated
 //                             into the K pool, v copied into the V pool.
+//   swl_qk_norm_rope_store_kv rows [q | k (| v)] of a projection whose biases are still to be added: per head bias, weighted RMS norm,
+//                             rotation; q times a factor per head into a buffer of its own, k into the K pool, and into the V
+//                             pool either the value columns or the KEYS AS PROJECTED (bias added, neither normed nor rotated).
 //   swl_latent_rope_store_kv  latent attention. Rows hold H query heads [d unrotated | dr rotated] and (optionally) the
 //                             compressed key/value row [r latent | dr shared rotated key part]. The rotated query parts go
 //                             to qa[t][h][r : r + dr] (the caller fills qa[t][h][0 : r] with the queries folded through
@@ -20,7 +24,9 @@
 //                             score maps over the same values.
 //   swl_head_gate             y[t][h][:] *= sigmoid(gate[t][h]).
 //
-// Pool layout as in qknorm_kv.hip: keys of a page [heads, 16, d], values transposed [heads, dv, 16].
+// Pool layout as in qknorm_kv.hip: keys of a page [heads, 16, d], values transposed [heads, dv, 16]. The two kernels in the
+// middle may lay heads out wider than they are (k_dim, v_dim: the row sizes that a compiled attention kernel serves); the
+// columns beyond the head are written as zeros, which neither scores nor outputs see.
 #include "swl_common.h"
 
 namespace swl {
@@ -29,11 +35,11 @@ constexpr int kRkThreads = 256;
 constexpr int kRkBlock = 16;        // tokens per KV block
 constexpr int kRkMaxPairs = 256;    // rot_dims <= 512
 
-__device__ __forceinline__ void rk_angles(float *cs, float *sn, const double *freq, int pos, int pairs) {
+__device__ __forceinline__ void rk_angles(float *cs, float *sn, const double *freq, int pos, int pairs, double mult = 1.0) {
     for (int i = threadIdx.x; i < pairs; i += kRkThreads) {
         const double a = static_cast<double>(pos) * freq[i];
-        cs[i] = static_cast<float>(cos(a));
-        sn[i] = static_cast<float>(sin(a));
+        cs[i] = static_cast<float>(cos(a) * mult);
+        sn[i] = static_cast<float>(sin(a) * mult);
     }
 }
 
@@ -82,26 +88,185 @@ __global__ __launch_bounds__(kRkThreads) void rope_store_kv_kernel(
 }
 
 template <typename T>
+__global__ __launch_bounds__(kRkThreads) void qk_norm_rope_store_kv_kernel(
+    const T *rows, T *q_out, const float *q_b, const float *k_b, const float *q_w, const float *k_w, const float *q_mult,
+    const double *freq, T *k_cache, T *v_cache, const int32_t *block_table, const int32_t *tok_seq, const int32_t *tok_pos, int nq,
+    int nk, int nv, int d, int dv, int rot_dims, int half, double rot_mult, int64_t tok_stride, int64_t q_out_stride, int k_dim,
+    int v_dim, int keys_as_values, int max_blocks_per_seq, int64_t block_stride, float eps) {
+    __shared__ float cs[kRkMaxPairs], sn[kRkMaxPairs];
+    const int64_t t = blockIdx.x;
+    const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
+    const int pos = tok_pos[t];
+    const int pairs = rot_dims >> 1;
+    rk_angles(cs, sn, freq, pos, pairs, rot_mult);
+    __syncthreads();
+    const T *row = rows + t * tok_stride;
+    T *qrow = q_out + t * q_out_stride;
+    const bool store = k_cache != nullptr;
+    int64_t blk = 0;
+    if (store) blk = block_table[static_cast<int64_t>(tok_seq[t]) * max_blocks_per_seq + pos / kRkBlock];
+    const int off = pos % kRkBlock;
+    T *kpage = k_cache + blk * block_stride, *vpage = v_cache + blk * block_stride;
+    const int heads = store ? nq + nk : nq;
+    bool wide = false;
+    if constexpr (sizeof(T) == 2) {
+        // 16-bit heads of a multiple of 8 elements up to 128 on 16-byte-aligned rows: a power-of-two group of lanes per head,
+        // 8 elements per lane; a rotated lane's partner elements are 8 neighbours too (or, interleaved, its own)
+        wide = d % 8 == 0 && d <= 128 && (tok_stride & 7) == 0 && (q_out_stride & 7) == 0 && (k_dim & 7) == 0 &&
+               (half ? (pairs & 7) == 0 : (rot_dims & 7) == 0) && (block_stride & 7) == 0 &&
+               ((reinterpret_cast<uintptr_t>(rows) | reinterpret_cast<uintptr_t>(q_out) | reinterpret_cast<uintptr_t>(k_cache) |
+                 reinterpret_cast<uintptr_t>(q_b) | reinterpret_cast<uintptr_t>(k_b) | reinterpret_cast<uintptr_t>(q_w) |
+                 reinterpret_cast<uintptr_t>(k_w)) & 15) == 0;
+        if (wide) {
+            const int lph = d <= 8 ? 1 : d <= 16 ? 2 : d <= 32 ? 4 : d <= 64 ? 8 : 16;      // lanes per head
+            const int hpw = 64 / lph;
+            const int slot = lane / lph, el = lane - slot * lph, e0 = el * 8;
+            auto load_biased = [&](float *v, const T *p, const float *b) {
+                const vec8_t<T> x = load8(p);
+#pragma unroll
+                for (int j = 0; j < 8; ++j) v[j] = to_f(x[j]);
+                if (b) {
+                    const float4_t b0 = *reinterpret_cast<const float4_t *>(b), b1 = *reinterpret_cast<const float4_t *>(b + 4);
+#pragma unroll
+                    for (int j = 0; j < 4; ++j) {
+                        v[j] += b0[j];
+                        v[4 + j] += b1[j];
+                    }
+                }
+            };
+            for (int hb = wave * hpw; hb < heads; hb += (kRkThreads / 64) * hpw) {
+                const int h = hb + slot;
+                const bool live = h < heads && e0 < d, is_q = h < nq;
+                const T *src = row + static_cast<int64_t>(live ? h : 0) * d;
+                const float *bias = is_q ? q_b : k_b, *wn = is_q ? q_w : k_w;
+                if (bias) bias += static_cast<int64_t>(live ? (is_q ? h : h - nq) : 0) * d;
+                float v[8];
+#pragma unroll
+                for (int j = 0; j < 8; ++j) v[j] = 0.f;
+                if (live) load_biased(v, src + e0, bias ? bias + e0 : nullptr);
+                float ss = 0.f;
+#pragma unroll
+                for (int j = 0; j < 8; ++j) ss += v[j] * v[j];
+                ss = lph == 1 ? ss : lph == 2 ? group_allreduce_sum<2>(ss) : lph == 4 ? group_allreduce_sum<4>(ss)
+                   : lph == 8 ? group_allreduce_sum<8>(ss) : group_allreduce_sum<16>(ss);
+                const float r = wn ? 1.0f / sqrtf(ss / static_cast<float>(d) + eps) : 1.0f;
+                if (!live) continue;
+                if (!is_q && keys_as_values) {
+                    T *dst = vpage + (static_cast<int64_t>(h - nq) * v_dim + e0) * kRkBlock + off;
+#pragma unroll
+                    for (int j = 0; j < 8; ++j) dst[j * kRkBlock] = to_t<T>(v[j]);
+                }
+                float n[8];
+#pragma unroll
+                for (int j = 0; j < 8; ++j) n[j] = wn ? v[j] * r * wn[e0 + j] : v[j];
+                if (e0 < rot_dims) {
+                    if (half) {
+                        const bool first = e0 < pairs;
+                        const int p0 = first ? e0 + pairs : e0 - pairs, a0 = first ? e0 : p0;
+                        float o[8];
+                        load_biased(o, src + p0, bias ? bias + p0 : nullptr);
+#pragma unroll
+                        for (int j = 0; j < 8; ++j) {
+                            const float w = wn ? o[j] * r * wn[p0 + j] : o[j];
+                            n[j] = first ? n[j] * cs[a0 + j] - w * sn[a0 + j] : n[j] * cs[a0 + j] + w * sn[a0 + j];
+                        }
+                    } else {
+#pragma unroll
+                        for (int j = 0; j < 8; j += 2) {
+                            const float c = cs[(e0 + j) >> 1], sv = sn[(e0 + j) >> 1], u = n[j], w = n[j + 1];
+                            n[j] = u * c - w * sv;
+                            n[j + 1] = w * c + u * sv;
+                        }
+                    }
+                }
+                const float mult = is_q && q_mult ? q_mult[h] : 1.0f;
+                vec8_t<T> o;
+#pragma unroll
+                for (int j = 0; j < 8; ++j) o[j] = to_t<T>(n[j] * mult);
+                store8(is_q ? qrow + static_cast<int64_t>(h) * k_dim + e0
+                            : kpage + (static_cast<int64_t>(h - nq) * kRkBlock + off) * k_dim + e0, o);
+            }
+        }
+    }
+    for (int h = wave; h < heads && !wide; h += kRkThreads / 64) {
+        const bool is_q = h < nq;
+        const T *src = row + static_cast<int64_t>(h) * d;
+        const float *bias = is_q ? q_b : k_b, *wn = is_q ? q_w : k_w;
+        if (bias) bias += static_cast<int64_t>(is_q ? h : h - nq) * d;
+        auto biased = [&](int e) { return to_f(src[e]) + (bias ? bias[e] : 0.f); };
+        float ss = 0.f;
+        for (int e = lane; e < d; e += 64) {
+            const float v = biased(e);
+            ss += v * v;
+            if (!is_q && keys_as_values) vpage[(static_cast<int64_t>(h - nq) * v_dim + e) * kRkBlock + off] = to_t<T>(v);
+        }
+        ss = wave_allreduce_sum(ss);
+        const float r = wn ? 1.0f / sqrtf(ss / static_cast<float>(d) + eps) : 1.0f;
+        auto normed = [&](int e) { return wn ? biased(e) * r * wn[e] : biased(e); };
+        const float mult = is_q && q_mult ? q_mult[h] : 1.0f;
+        T *dst = is_q ? qrow + static_cast<int64_t>(h) * k_dim : kpage + (static_cast<int64_t>(h - nq) * kRkBlock + off) * k_dim;
+        for (int e = lane; e < d; e += 64) {
+            float n = normed(e);
+            if (e < rot_dims) {
+                const bool first = half ? e < pairs : (e & 1) == 0;
+                const int p = half ? (first ? e + pairs : e - pairs) : e ^ 1, a = half ? (first ? e : p) : e >> 1;
+                const float w = normed(p);
+                n = first ? n * cs[a] - w * sn[a] : n * cs[a] + w * sn[a];
+            }
+            dst[e] = to_t<T>(n * mult);
+        }
+    }
+    // zero the columns beyond the head
+    const int kpad = k_dim - d;
+    for (int i = threadIdx.x; i < heads * kpad; i += kRkThreads) {
+        const int h = i / kpad, e = d + i - h * kpad;
+        if (h < nq) qrow[static_cast<int64_t>(h) * k_dim + e] = to_t<T>(0.f);
+        else kpage[(static_cast<int64_t>(h - nq) * kRkBlock + off) * k_dim + e] = to_t<T>(0.f);
+    }
+    if (!store) return;
+    const int nval = keys_as_values ? nk : nv, dval = keys_as_values ? d : dv, vpad = v_dim - dval;
+    if (!keys_as_values) {
+        const T *vrow = row + static_cast<int64_t>(nq + nk) * d;
+        for (int i = threadIdx.x; i < nv * dv; i += kRkThreads) {
+            const int g = i / dv, c = i - g * dv;
+            vpage[(static_cast<int64_t>(g) * v_dim + c) * kRkBlock + off] = vrow[i];
+        }
+    }
+    for (int i = threadIdx.x; i < nval * vpad; i += kRkThreads) {
+        const int g = i / vpad, c = dval + i - g * vpad;
+        vpage[(static_cast<int64_t>(g) * v_dim + c) * kRkBlock + off] = to_t<T>(0.f);
+    }
+}
+
+template <typename T>
 __global__ __launch_bounds__(kRkThreads) void latent_rope_store_kv_kernel(
     const T *proj, T *qa, const double *freq, const float *c_w, T *k_cache, T *v_cache, const int32_t *block_table,
     const int32_t *tok_seq, const int32_t *tok_pos, int H, int d, int dr, int r, int64_t proj_stride, int64_t dkv_col,
-    int64_t qa_stride, int max_blocks_per_seq, int64_t block_stride, float eps) {
+    int64_t qa_stride, int max_blocks_per_seq, int64_t block_stride, float eps, int half, double rot_mult, int k_dim,
+    int v_dim) {
     __shared__ float cs[kRkMaxPairs], sn[kRkMaxPairs];
     __shared__ float red[kRkThreads / 64];
     const int64_t t = blockIdx.x;
     const int pos = tok_pos[t];
     const int pairs = dr >> 1;
-    rk_angles(cs, sn, freq, pos, pairs);
+    rk_angles(cs, sn, freq, pos, pairs, rot_mult);
     __syncthreads();
     const T *row = proj + t * proj_stride;
     T *qrow = qa + t * qa_stride;
+    // pair j of a rotated part: elements (2j, 2j + 1), or (j, j + pairs)
+    const int step = half ? 1 : 2, gap = half ? pairs : 1;
     for (int i = threadIdx.x; i < H * pairs; i += kRkThreads) {
         const int h = i / pairs, j = i - h * pairs;
-        const T *p = row + static_cast<int64_t>(h) * (d + dr) + d + 2 * j;
-        T *o = qrow + static_cast<int64_t>(h) * (r + dr) + r + 2 * j;
-        const float u = to_f(p[0]), v = to_f(p[1]);
+        const T *p = row + static_cast<int64_t>(h) * (d + dr) + d + step * j;
+        T *o = qrow + static_cast<int64_t>(h) * k_dim + r + step * j;
+        const float u = to_f(p[0]), v = to_f(p[gap]);
         o[0] = to_t<T>(u * cs[j] - v * sn[j]);
-        o[1] = to_t<T>(v * cs[j] + u * sn[j]);
+        o[gap] = to_t<T>(v * cs[j] + u * sn[j]);
+    }
+    const int kpad = k_dim - r - dr, vpad = v_dim - r;
+    for (int i = threadIdx.x; i < H * kpad; i += kRkThreads) {
+        const int h = i / kpad;
+        qrow[static_cast<int64_t>(h) * k_dim + r + dr + i - h * kpad] = to_t<T>(0.f);
     }
     if (dkv_col < 0 || k_cache == nullptr) return;
     const T *z = row + dkv_col;
@@ -119,7 +284,7 @@ __global__ __launch_bounds__(kRkThreads) void latent_rope_store_kv_kernel(
     const float rinv = 1.0f / sqrtf(ss / static_cast<float>(r) + eps);
     const int64_t blk = block_table[static_cast<int64_t>(tok_seq[t]) * max_blocks_per_seq + pos / kRkBlock];
     const int off = pos % kRkBlock;
-    T *kdst = k_cache + blk * block_stride + static_cast<int64_t>(off) * (r + dr);
+    T *kdst = k_cache + blk * block_stride + static_cast<int64_t>(off) * k_dim;
     T *vdst = v_cache + blk * block_stride + off;
     for (int i = threadIdx.x; i < r; i += kRkThreads) {
         const T c = to_t<T>(to_f(z[i]) * rinv * c_w[i]);
@@ -127,10 +292,12 @@ __global__ __launch_bounds__(kRkThreads) void latent_rope_store_kv_kernel(
         vdst[static_cast<int64_t>(i) * kRkBlock] = c;
     }
     for (int j = threadIdx.x; j < pairs; j += kRkThreads) {
-        const float u = to_f(z[r + 2 * j]), v = to_f(z[r + 2 * j + 1]);
-        kdst[r + 2 * j] = to_t<T>(u * cs[j] - v * sn[j]);
-        kdst[r + 2 * j + 1] = to_t<T>(v * cs[j] + u * sn[j]);
+        const float u = to_f(z[r + step * j]), v = to_f(z[r + step * j + gap]);
+        kdst[r + step * j] = to_t<T>(u * cs[j] - v * sn[j]);
+        kdst[r + step * j + gap] = to_t<T>(v * cs[j] + u * sn[j]);
     }
+    for (int i = threadIdx.x; i < kpad; i += kRkThreads) kdst[r + dr + i] = to_t<T>(0.f);
+    for (int i = threadIdx.x; i < vpad; i += kRkThreads) vdst[static_cast<int64_t>(r + i) * kRkBlock] = to_t<T>(0.f);
 }
 
 template <typename T>
@@ -155,6 +322,18 @@ __global__ __launch_bounds__(256) void diff_head_combine_kernel(T *out, const fl
 template <typename T>
 __global__ __launch_bounds__(256) void head_gate_kernel(T *y, const T *gate, int64_t gate_stride, int H, int dv) {
     const int64_t t = blockIdx.x;
+    if constexpr (sizeof(T) == 2) {
+        if ((dv & 7) == 0 && (reinterpret_cast<uintptr_t>(y) & 15) == 0) {      // 8 columns of one head per lane
+            for (int i = threadIdx.x * 8; i < H * dv; i += 256 * 8) {
+                const float g = rk_sigmoid(to_f(gate[t * gate_stride + i / dv]));
+                vec8_t<T> v = load8(y + t * H * dv + i);
+#pragma unroll
+                for (int j = 0; j < 8; ++j) v[j] = to_t<T>(to_f(v[j]) * g);
+                store8(y + t * H * dv + i, v);
+            }
+            return;
+        }
+    }
     for (int i = threadIdx.x; i < H * dv; i += 256) {
         const float g = rk_sigmoid(to_f(gate[t * gate_stride + i / dv]));
         y[t * H * dv + i] = to_t<T>(to_f(y[t * H * dv + i]) * g);
@@ -185,15 +364,44 @@ extern "C" int swl_rope_store_kv(void *qkv, const double *freq, void *k_cache, v
     return swl::check_launch();
 }
 
+extern "C" int swl_qk_norm_rope_store_kv(const void *rows, void *q_out, const float *q_b, const float *k_b, const float *q_w,
+                                         const float *k_w, const float *q_mult, const double *freq, void *k_cache, void *v_cache,
+                                         const int32_t *block_table, const int32_t *tok_seq, const int32_t *tok_pos,
+                                         int64_t num_tokens, int32_t num_q_heads, int32_t num_k_heads, int32_t num_v_heads,
+                                         int32_t dim, int32_t vdim, int32_t rot_dims, int32_t half, double rot_mult,
+                                         int64_t tok_stride, int64_t q_out_stride, int32_t k_dim, int32_t v_dim,
+                                         int32_t keys_as_values, int32_t max_blocks_per_seq, int64_t block_stride, float eps,
+                                         int32_t dtype, swl_stream_t stream) {
+    if (num_tokens < 0 || num_q_heads <= 0 || num_k_heads < 0 || num_v_heads < 0 || dim <= 0 || vdim <= 0) return SWL_ERR_BAD_ARG;
+    if (rot_dims < 0 || (rot_dims & 1) || rot_dims > dim || (!half && (dim & 1))) return SWL_ERR_BAD_ARG;
+    if (keys_as_values && (num_v_heads != 0 || vdim != dim)) return SWL_ERR_BAD_ARG;
+    if (k_dim < dim || v_dim < vdim || q_out_stride < static_cast<int64_t>(num_q_heads) * k_dim) return SWL_ERR_BAD_ARG;
+    if (tok_stride < static_cast<int64_t>(num_q_heads + num_k_heads) * dim + static_cast<int64_t>(num_v_heads) * vdim)
+        return SWL_ERR_BAD_ARG;
+    if (num_tokens == 0) return SWL_OK;
+    if (!rows || !q_out || rows == q_out || !tok_pos || (rot_dims > 0 && !freq)) return SWL_ERR_BAD_ARG;
+    if (k_cache && (!v_cache || !block_table || !tok_seq || max_blocks_per_seq <= 0)) return SWL_ERR_BAD_ARG;
+    if (num_tokens > 0x7fffffffLL || rot_dims > 2 * swl::kRkMaxPairs) return SWL_ERR_UNSUPPORTED;
+    SWL_DISPATCH_DTYPE3(dtype, T, {
+        hipLaunchKernelGGL((swl::qk_norm_rope_store_kv_kernel<T>), dim3(static_cast<unsigned>(num_tokens)), dim3(swl::kRkThreads),
+                           0, static_cast<hipStream_t>(stream), static_cast<const T *>(rows), static_cast<T *>(q_out), q_b, k_b,
+                           q_w, k_w, q_mult, freq, static_cast<T *>(k_cache), static_cast<T *>(v_cache), block_table, tok_seq,
+                           tok_pos, num_q_heads, num_k_heads, num_v_heads, dim, vdim, rot_dims, half, rot_mult, tok_stride,
+                           q_out_stride, k_dim, v_dim, keys_as_values, max_blocks_per_seq, block_stride, eps);
+    });
+    return swl::check_launch();
+}
+
 extern "C" int swl_latent_rope_store_kv(const void *proj, void *qa, const double *freq, const float *c_norm, void *k_cache,
                                         void *v_cache, const int32_t *block_table, const int32_t *tok_seq,
                                         const int32_t *tok_pos, int64_t num_tokens, int32_t num_heads, int32_t dim,
                                         int32_t rot_dim, int32_t kv_rank, int64_t proj_stride, int64_t dkv_col,
                                         int64_t qa_stride, int32_t max_blocks_per_seq, int64_t block_stride, float eps,
-                                        int32_t dtype, swl_stream_t stream) {
+                                        int32_t half, double rot_mult, int32_t k_dim, int32_t v_dim, int32_t dtype,
+                                        swl_stream_t stream) {
     if (num_tokens < 0 || num_heads <= 0 || dim <= 0 || rot_dim <= 0 || (rot_dim & 1) || kv_rank <= 0) return SWL_ERR_BAD_ARG;
-    if (proj_stride < static_cast<int64_t>(num_heads) * (dim + rot_dim) ||
-        qa_stride < static_cast<int64_t>(num_heads) * (kv_rank + rot_dim))
+    if (k_dim < kv_rank + rot_dim || v_dim < kv_rank) return SWL_ERR_BAD_ARG;
+    if (proj_stride < static_cast<int64_t>(num_heads) * (dim + rot_dim) || qa_stride < static_cast<int64_t>(num_heads) * k_dim)
         return SWL_ERR_BAD_ARG;
     if (dkv_col >= 0 && dkv_col + kv_rank + rot_dim > proj_stride) return SWL_ERR_BAD_ARG;
     if (num_tokens == 0) return SWL_OK;
@@ -206,7 +414,7 @@ extern "C" int swl_latent_rope_store_kv(const void *proj, void *qa, const double
                            dim3(swl::kRkThreads), 0, static_cast<hipStream_t>(stream), static_cast<const T *>(proj),
                            static_cast<T *>(qa), freq, c_norm, static_cast<T *>(k_cache), static_cast<T *>(v_cache),
                            block_table, tok_seq, tok_pos, num_heads, dim, rot_dim, kv_rank, proj_stride, dkv_col, qa_stride,
-                           max_blocks_per_seq, block_stride, eps);
+                           max_blocks_per_seq, block_stride, eps, half, rot_mult, k_dim, v_dim);
     });
     return swl::check_launch();
 }

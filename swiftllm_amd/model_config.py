@@ -2,6 +2,7 @@
 
 Mirrors swiftllm/model_config.py:5-46 (attribute names, defaults, kv-slot size formula)."""
 import json
+import math
 import os
 
 import torch
@@ -106,6 +107,17 @@ class LayerRun:
         self.index, self.layer, self.pass_index = index, layer, pass_index
 
 
+def looped_layer_runs(num_layers: int, loop: dict):
+    """LayerRuns of a stack in which layers start .. stop - 1 run `times` times in a row (loop None: every layer once)."""
+    start, stop, times = (int(loop[k]) for k in ("start", "stop", "times")) if loop else (0, 0, 0)
+    if loop and not (0 <= start < stop <= num_layers and times >= 1):
+        raise ValueError(f"bad loop {loop!r} for {num_layers} layers")
+    order = [(i, -1) for i in range(start)]
+    order += [(i, t if i == start else -1) for t in range(times) for i in range(start, stop)]
+    order += [(i, -1) for i in range(stop, num_layers)]
+    return [LayerRun(n, layer, t) for n, (layer, t) in enumerate(order)]
+
+
 class KekapelModelConfig:
     """Kekapel: a decoder-only model with learned positions, sandwich LayerNorms around every sublayer, sliding-window
     attention with q/k norm, tanh soft-capping and pre-softmax head mixing, dense (PolyNorm) or mixture-of-experts
@@ -124,21 +136,8 @@ class KekapelModelConfig:
         self.layers = [KekapelLayerConfig(layer) for layer in model_config["layers"]]
         self.num_layers = len(self.layers)
         loop = model_config.get("loop")
-        if loop:
-            self.loop_start, self.loop_stop, self.loop_times = int(loop["start"]), int(loop["stop"]), int(loop["times"])
-            if not (0 <= self.loop_start < self.loop_stop <= self.num_layers and self.loop_times >= 1):
-                raise ValueError(f"bad loop {loop!r} for {self.num_layers} layers")
-        else:
-            self.loop_start = self.loop_stop = self.loop_times = 0
-        self.layer_runs = []
-        order = list(range(self.loop_start))
-        for t in range(self.loop_times):
-            order += [(i, t) for i in range(self.loop_start, self.loop_stop)]
-        order += list(range(self.loop_stop, self.num_layers))
-        for item in order:
-            layer, t = item if isinstance(item, tuple) else (item, -1)
-            first = t >= 0 and layer == self.loop_start
-            self.layer_runs.append(LayerRun(len(self.layer_runs), layer, t if first else -1))
+        self.loop_times = int(loop["times"]) if loop else 0
+        self.layer_runs = looped_layer_runs(self.num_layers, loop)
         self.num_layer_runs = len(self.layer_runs)
         # what the scheduler-facing code reads off any model's configuration
         self.num_q_heads = max(l.mixer.num_q_heads for l in self.layers)
@@ -163,7 +162,6 @@ class KekapelModelConfig:
 def distance_bias_rows(table_rows: int, far: float, max_distance: int):
     """Row of a learned distance-bias table for every distance 0 .. max_distance - 1: the first table_rows // 2 distances have
     a row each, beyond that the rows advance in equal steps of log(distance) and the last row is reached at `far`."""
-    import math
     half = table_rows // 2
     rows = []
     for dist in range(max_distance):
@@ -331,18 +329,37 @@ class LorulixModelConfig:
 
 # ---- Rosilix ---------------------------------------------------------------------------------------------------------------
 class RotaryConfig:
-    """Rotary positions on interleaved pairs: dimension 2i of a head turns with dimension 2i + 1 by the angle
-    position * base^(-2i / dims), for i < dims / 2; the dimensions from `dims` on pass unchanged."""
+    """Rotary positions on the first `dims` dimensions of a head; the dimensions from `dims` on pass unchanged. half = False:
+    dimension 2i turns with dimension 2i + 1 (interleaved pairs); half = True: dimension i turns with dimension i + dims / 2. The
+    angle is position * base^(-2i / dims), i < dims / 2. `scaling` (factor, original, fast, slow) interpolates by parts (YaRN):
+    dimensions that turn fewer than `slow` times over `original` positions are slowed down by `factor`, those that turn more than
+    `fast` times are kept, a linear ramp lies between; cosines and sines are then multiplied by 0.1 ln(factor) + 1."""
 
-    def __init__(self, rot: dict, head_dim: int):
+    def __init__(self, rot: dict, head_dim: int, half: bool = False):
         self.dims = int(rot["dims"]) if rot else 0
         self.base = float(rot["base"]) if rot else 1.0
+        self.half = half
+        self.multiplier = 1.0
+        self.scaling = None
+        scaling = (rot or {}).get("scaling")
+        if scaling and self.dims:
+            self.scaling = tuple(float(scaling[k]) for k in ("factor", "original", "fast", "slow"))
+            self.multiplier = 0.1 * math.log(self.scaling[0]) + 1.0
         if self.dims < 0 or self.dims % 2 or self.dims > head_dim:
             raise ValueError(f"rot.dims ({self.dims}) must be even and at most the head size ({head_dim})")
 
     def frequencies(self):
-        """base^(-2i / dims) for i < dims / 2, in float64."""
-        return [self.base ** (-2.0 * i / self.dims) for i in range(self.dims // 2)]
+        """The angle per position of each of the dims / 2 pairs, in float64."""
+        plain = [self.base ** (-2.0 * i / self.dims) for i in range(self.dims // 2)]
+        if self.scaling is None:
+            return plain
+        factor, original, fast, slow = self.scaling
+
+        def dim_of(turns):      # the (fractional) pair index that turns this often over `original` positions
+            return self.dims * math.log(original / (2.0 * math.pi * turns)) / (2.0 * math.log(self.base))
+        lo, hi = max(math.floor(dim_of(fast)), 0), min(math.ceil(dim_of(slow)), self.dims - 1)
+        ramps = [min(max((i - lo) / max(hi - lo, 0.001), 0.0), 1.0) for i in range(self.dims // 2)]
+        return [f / factor * r + f * (1.0 - r) for f, r in zip(plain, ramps)]
 
 
 class RosilixDiffAttentionConfig:
@@ -671,3 +688,170 @@ class RatilornModelConfig:
     def load_from_model_path(model_path: str) -> "RatilornModelConfig":
         with open(os.path.join(model_path, "config.json"), "r", encoding="utf-8") as f:
             return RatilornModelConfig(json.load(f))
+
+
+# ---- Rokevik ---------------------------------------------------------------------------------------------------------------
+class RokevikAttentionConfig:
+    """Softmax attention over every earlier key whose values are the projected keys themselves (before their norm and
+    rotation): biased projections, weighted per-head q/k norm, rotate-half rotary, a temperature per head, tanh soft-capping and
+    a gate per head."""
+    kind = "attention"
+
+    def __init__(self, mixer: dict):
+        self.num_q_heads = int(mixer["heads"])
+        self.num_kv_heads = int(mixer.get("kv_heads", self.num_q_heads))
+        self.head_dim = int(mixer["dim"])
+        self.value_dim = int(mixer.get("vdim", self.head_dim))
+        self.scale = float(mixer["scale"])
+        cap = mixer.get("softcap")
+        self.softcap = float(cap) if cap else 0.0           # 0: scores are not capped
+        self.rot = RotaryConfig(mixer.get("rot"), self.head_dim, half=True)
+        if self.num_q_heads % self.num_kv_heads:
+            raise ValueError(f"heads ({self.num_q_heads}) must be a multiple of kv_heads ({self.num_kv_heads})")
+        if self.value_dim != self.head_dim:
+            raise ValueError(f"the values are the keys: vdim ({self.value_dim}) must equal dim ({self.head_dim})")
+
+    @property
+    def q_size(self) -> int:
+        return self.num_q_heads * self.head_dim
+
+    @property
+    def k_size(self) -> int:
+        return self.num_kv_heads * self.head_dim
+
+    @property
+    def v_size(self) -> int:
+        return self.num_kv_heads * self.value_dim
+
+    @property
+    def o_size(self) -> int:
+        return self.num_q_heads * self.value_dim
+
+
+class RokevikLatentAttentionConfig:
+    """Latent attention inside a sliding window: keys and values of all heads are up-projections of one cached latent row of
+    `kv_rank` per token, plus one rotated key part of `rot_dim` shared by the heads; the heads are gated."""
+    kind = "latent_attention"
+
+    def __init__(self, mixer: dict):
+        self.num_q_heads = int(mixer["heads"])
+        self.num_kv_heads = 1
+        self.head_dim = int(mixer["dim"])                       # unrotated part of a query / key head
+        self.rot_dim = int(mixer["rot_dim"])
+        self.value_dim = int(mixer.get("vdim", self.head_dim))
+        self.kv_rank = int(mixer["kv_rank"])
+        self.scale = float(mixer["scale"])
+        mask = mixer.get("mask") or {}
+        self.window = int(mask["size"]) if mask.get("size") else 0     # 0: every earlier key is visible
+        self.rot = RotaryConfig(mixer["rot"], self.rot_dim, half=True)
+        if self.rot.dims != self.rot_dim:
+            raise ValueError(f"rot.dims ({self.rot.dims}) must equal rot_dim ({self.rot_dim})")
+
+    @property
+    def q_size(self) -> int:
+        return self.num_q_heads * (self.head_dim + self.rot_dim)
+
+    @property
+    def dkv_size(self) -> int:
+        return self.kv_rank + self.rot_dim
+
+    @property
+    def k_size(self) -> int:
+        """Elements of the cached key row: the latent and the shared rotated part."""
+        return self.kv_rank + self.rot_dim
+
+    @property
+    def v_size(self) -> int:
+        """Elements of the cached value row: the latent once more (kept transposed for the value product)."""
+        return self.kv_rank
+
+    @property
+    def o_size(self) -> int:
+        return self.num_q_heads * self.value_dim
+
+
+class MinGruConfig:
+    """minGRU: `width` independent fp32 states per sequence, gate and candidate read from the current token only."""
+    kind = "mingru"
+
+    def __init__(self, mixer: dict):
+        self.width = int(mixer["width"])
+        if self.width < 1:
+            raise ValueError(f"mingru width must be positive, got {self.width}")
+
+
+class RokevikMlpConfig:
+    """`moe`: SiLU gated experts behind a sigmoid router whose scores multiply the experts' INPUTS, plus an optional shared
+    expert."""
+
+    def __init__(self, mlp: dict):
+        self.kind = mlp["kind"]
+        if self.kind != "moe":
+            raise ValueError(f"unsupported mlp.kind {self.kind!r}")
+        self.ffn_inter_dim = int(mlp["expert"]["ff"])
+        self.num_experts = int(mlp["router"]["experts"])
+        self.top_k = int(mlp["router"]["top"])
+        self.shared_ffn_inter_dim = int(mlp["shared"]["ff"]) if mlp.get("shared") else 0
+        if not 0 < self.top_k <= self.num_experts:
+            raise ValueError(f"router.top ({self.top_k}) must be in 1..experts ({self.num_experts})")
+
+
+class RokevikLayerConfig:
+    MIXERS = {m.kind: m for m in (RokevikAttentionConfig, RokevikLatentAttentionConfig, MinGruConfig)}
+
+    def __init__(self, layer: dict):
+        self.type = layer["type"]
+        if self.type not in self.MIXERS:
+            raise ValueError(f"unsupported layer type {self.type!r}")
+        self.mixer = self.MIXERS[self.type](layer["mixer"])
+        self.mlp = RokevikMlpConfig(layer["mlp"]) if layer.get("mlp") else None
+
+
+class RokevikModelConfig:
+    """Rokevik: a decoder-only model whose residual is several fp32 streams (hyper-connections: every sublayer reads a weighted
+    sum of them and writes back into each, while a small matrix mixes them), RMS norms in groups in front of every sublayer,
+    three kinds of mixer in any order (keys-as-values attention, windowed latent attention, minGRU), mixture-of-experts
+    feed-forwards, a span of layers that runs several times, and capped logits. Every size and constant is read from
+    config.json. `streams` absent: one plain residual. The design has no position table: `max_positions`, if config.json gives
+    it, bounds a sequence; otherwise the bound is DEFAULT_MAX_POSITIONS."""
+    DEFAULT_MAX_POSITIONS = 1 << 20
+
+    def __init__(self, model_config: dict):
+        if model_config.get("architecture") != "Rokevik":
+            raise AssertionError(f"unsupported architecture {model_config.get('architecture')!r}")
+        self.vocab_size = int(model_config["vocab"])
+        self.hidden_size = int(model_config["width"])
+        self.max_position_embeddings = int(model_config.get("max_positions") or self.DEFAULT_MAX_POSITIONS)
+        self.norm_eps = float(model_config["norm"]["eps"])
+        self.norm_groups = int(model_config["norm"].get("groups", 1))
+        if self.norm_groups < 1 or self.hidden_size % self.norm_groups:
+            raise ValueError(f"width ({self.hidden_size}) must be a multiple of norm.groups ({self.norm_groups})")
+        self.num_streams = int(model_config.get("streams") or 0)        # 0: a plain residual, no stream weights
+        cap = model_config.get("logit_softcap")
+        self.logit_softcap = float(cap) if cap else 0.0
+        self.layers = [RokevikLayerConfig(layer) for layer in model_config["layers"]]
+        self.num_layers = len(self.layers)
+        self.layer_runs = looped_layer_runs(self.num_layers, model_config.get("loop"))
+        self.num_layer_runs = len(self.layer_runs)
+        attn = [l.mixer for l in self.layers if l.type != "mingru"]
+        # what the scheduler-facing code reads off any model's configuration
+        self.num_q_heads = max((m.num_q_heads for m in attn), default=1)
+        self.num_kv_heads = max((m.num_kv_heads for m in attn), default=1)
+        self.head_dim = max((m.head_dim for m in attn), default=1)
+
+    @property
+    def has_state(self) -> bool:
+        return any(l.type == "mingru" for l in self.layers)
+
+    def kv_elems_per_token(self) -> int:
+        """Cached elements per token over all layer runs with a cache (a looped layer has one per pass)."""
+        mixers = [self.layers[r.layer].mixer for r in self.layer_runs]
+        return sum(m.k_size + m.v_size for m in mixers if m.kind != "mingru")
+
+    def get_kvslot_size(self, dtype: torch.dtype = torch.bfloat16) -> int:
+        return max(self.kv_elems_per_token(), 1) * dtype.itemsize
+
+    @staticmethod
+    def load_from_model_path(model_path: str) -> "RokevikModelConfig":
+        with open(os.path.join(model_path, "config.json"), "r", encoding="utf-8") as f:
+            return RokevikModelConfig(json.load(f))

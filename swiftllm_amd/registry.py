@@ -15,6 +15,7 @@ MODELS = {
     "Lorulix": ("swiftllm_amd.model_config:LorulixModelConfig", "swiftllm_amd.worker.lorulix_model:LorulixModel"),
     "Rosilix": ("swiftllm_amd.model_config:RosilixModelConfig", "swiftllm_amd.worker.rosilix_model:RosilixModel"),
     "Ratilorn": ("swiftllm_amd.model_config:RatilornModelConfig", "swiftllm_amd.worker.ratilorn_model:RatilornModel"),
+    "Rokevik": ("swiftllm_amd.model_config:RokevikModelConfig", "swiftllm_amd.worker.rokevik_model:RokevikModel"),
 }
 
 

@@ -166,10 +166,16 @@ class StepPlan:
     tok_start: np.ndarray = None        # [T] int32 position of the first token of the token's portion
     # [T] int32 state slot * 2 + tail parity of the token's sequence; zeros until a worker with per-sequence state fills it
     tok_state: np.ndarray = None
+    # the portions cut into runs of up to CHUNK tokens (what a recurrence that is linear in its state evaluates in parallel), and
+    # the first of each sequence's
+    chunk_row0: np.ndarray = None       # [NC] int32 first token row of each chunk
+    chunk_cnt: np.ndarray = None        # [NC] int32 tokens in it
+    seq_chunk0: np.ndarray = None       # [S] int32
 
     TILE = 16
+    CHUNK = 32
     SEGMENTS = ("input_ids", "tok_pos", "tok_seq", "want_rows", "tile_row0", "tile_cnt", "seq_row0", "seq_cnt", "tok_start",
-                "tok_state")
+                "tok_state", "chunk_row0", "chunk_cnt", "seq_chunk0")
 
     def packed_layout(self):
         out, off = [], 0
@@ -216,16 +222,24 @@ def plan_step(entries: Sequence[StepEntry], vocab_size: int = None, max_position
         targets.append(int(e.start + n))
         base += n
     cat = (lambda xs: np.concatenate(xs) if xs else np.empty(0, dtype=np.int32))
-    row0, cnt, at = [], [], 0
-    for e in entries:
-        n = len(e.tokens)
-        starts = np.arange(0, n, StepPlan.TILE, dtype=np.int32)
-        row0.append(at + starts)
-        cnt.append(np.minimum(StepPlan.TILE, n - starts).astype(np.int32))
-        at += n
+
+    def runs_of(size):
+        """(first rows, counts) of the portions cut into runs of up to `size` tokens"""
+        row0, cnt, at = [], [], 0
+        for e in entries:
+            n = len(e.tokens)
+            starts = np.arange(0, n, size, dtype=np.int32)
+            row0.append(at + starts)
+            cnt.append(np.minimum(size, n - starts).astype(np.int32))
+            at += n
+        return cat(row0), cat(cnt)
+    tile_row0, tile_cnt = runs_of(StepPlan.TILE)
+    chunk_row0, chunk_cnt = runs_of(StepPlan.CHUNK)
     counts = np.asarray([len(e.tokens) for e in entries], dtype=np.int32)
     starts = np.asarray([e.start for e in entries], dtype=np.int32)
-    return StepPlan(tile_row0=cat(row0), tile_cnt=cat(cnt), seq_cnt=counts,
+    chunks = -(-counts // StepPlan.CHUNK)
+    return StepPlan(tile_row0=tile_row0, tile_cnt=tile_cnt, seq_cnt=counts, chunk_row0=chunk_row0, chunk_cnt=chunk_cnt,
+                    seq_chunk0=(np.cumsum(chunks) - chunks).astype(np.int32),
                     seq_row0=(np.cumsum(counts) - counts).astype(np.int32), tok_start=np.repeat(starts, counts),
                     tok_state=np.zeros(base, dtype=np.int32),
                     num_tokens=base, num_seqs=len(seq_ids), seq_ids_list=seq_ids, target_lens_list=targets,

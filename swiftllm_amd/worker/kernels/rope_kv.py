@@ -1,4 +1,4 @@
-"""Rotary positions on interleaved pairs fused with the paged KV store (plain heads, and the compressed rows of latent
+"""Rotary positions fused with the paged KV store (plain heads, heads with biases and a q/k norm, the compressed rows of latent
 attention), and the per-head steps after the softmax: the combination of two score maps, the head gate. csrc/rope_kv.hip."""
 import torch
 
@@ -41,16 +41,51 @@ def rope_and_store_kv(qkv: torch.Tensor, freq: torch.Tensor, rot_dims: int, pool
               stride, _hip.dtype_code3(qkv.dtype), _hip.stream())
 
 
+def qk_norm_rope_and_store_kv(rows: torch.Tensor, q_b: torch.Tensor, k_b: torch.Tensor, q_norm: torch.Tensor,
+                              k_norm: torch.Tensor, q_mult: torch.Tensor, freq: torch.Tensor, rot, pool: torch.Tensor,
+                              pool_slice: PoolSlice, block_table: torch.Tensor, tok_seq: torch.Tensor, tok_pos: torch.Tensor,
+                              num_q_heads: int, num_k_heads: int, num_v_heads: int, dim: int, vdim: int, eps: float,
+                              k_dim: int = 0, v_dim: int = 0) -> torch.Tensor:
+    """rows [q | k | v (| anything)] of one fused projection whose biases (fp32, optional) are still to be added -> the queries
+    [T, num_q_heads * k_dim]: biased, RMS-normed per head (fp32 weights of `dim` shared by the heads, None: not normed), rotated as
+    `rot` (a RotaryConfig) says and multiplied by q_mult[head] (None: 1). The keys go to the pool likewise; the values to the V
+    pool — with num_v_heads = 0 the rows hold none and the biased keys, neither normed nor rotated, are the values. k_dim / v_dim:
+    row sizes in the pool and in the result (default dim / vdim), columns beyond the head zero. pool None: queries only."""
+    _hip.require_gpu_tensor(rows, "rows")
+    n = rows.shape[0]
+    k_dim, v_dim = k_dim or dim, v_dim or vdim
+    assert rows.dim() == 2 and rows.stride(1) == 1 and tok_pos.dtype == torch.int32 and tok_pos.shape[0] == n
+    assert rows.shape[1] >= (num_q_heads + num_k_heads) * dim + num_v_heads * vdim
+    for t, size in ((q_b, num_q_heads * dim), (k_b, num_k_heads * dim), (q_norm, dim), (k_norm, dim), (q_mult, num_q_heads)):
+        assert t is None or (t.dtype == torch.float32 and t.is_contiguous() and t.numel() == size)
+    rot_dims = rot.dims if freq is not None else 0
+    assert freq is None or (freq.dtype == torch.float64 and freq.numel() == rot_dims // 2)
+    kp, vp, stride = _pool_ptrs(pool, pool_slice)
+    if pool is not None:
+        assert pool.dtype == rows.dtype and block_table.is_contiguous() and tok_seq.dtype == torch.int32
+    q = torch.empty((n, num_q_heads * k_dim), dtype=rows.dtype, device=rows.device)
+    _hip.call("swl_qk_norm_rope_store_kv", _hip.ptr(rows), _hip.ptr(q), _hip.ptr(q_b), _hip.ptr(k_b), _hip.ptr(q_norm),
+              _hip.ptr(k_norm), _hip.ptr(q_mult), _hip.ptr(freq), kp, vp, _hip.ptr(block_table), _hip.ptr(tok_seq),
+              _hip.ptr(tok_pos), n, num_q_heads, num_k_heads, num_v_heads, dim, vdim, rot_dims, 1 if rot.half else 0,
+              float(rot.multiplier), rows.stride(0), q.stride(0), k_dim, v_dim, 1 if num_v_heads == 0 else 0,
+              block_table.shape[1] if block_table is not None else 0, stride, float(eps), _hip.dtype_code3(rows.dtype),
+              _hip.stream())
+    return q
+
+
 def latent_rope_and_store_kv(proj: torch.Tensor, qa: torch.Tensor, freq: torch.Tensor, c_norm: torch.Tensor,
                              pool: torch.Tensor, pool_slice: PoolSlice, block_table: torch.Tensor, tok_seq: torch.Tensor,
-                             tok_pos: torch.Tensor, mixer, dkv_col: int, eps: float):
+                             tok_pos: torch.Tensor, mixer, dkv_col: int, eps: float, k_dim: int = 0, v_dim: int = 0):
     """proj rows: the query heads [dim | rot_dim] and, at column dkv_col (< 0: the layer reads another layer's cache), the
-    compressed row [kv_rank | rot_dim]. Writes the rotated query parts into qa [T, heads, kv_rank + rot_dim] (columns from
-    kv_rank on) and the normed latent + rotated shared key part into the pool."""
+    compressed row [kv_rank | rot_dim]. Writes the rotated query parts into qa [T, heads, k_dim] (columns kv_rank .. kv_rank +
+    rot_dim) and the normed latent + rotated shared key part into the pool. The layout of the pairs and the multiplier of the
+    rotation are mixer.rot's. k_dim / v_dim: row sizes in qa and in the pool (default kv_rank + rot_dim / kv_rank), columns beyond
+    zeroed."""
     _hip.require_gpu_tensor(proj, "proj")
     n = proj.shape[0]
+    k_dim, v_dim = k_dim or mixer.kv_rank + mixer.rot_dim, v_dim or mixer.kv_rank
     assert proj.dim() == 2 and proj.stride(1) == 1 and qa.is_contiguous() and qa.dtype == proj.dtype
-    assert qa.shape == (n, mixer.num_q_heads * (mixer.kv_rank + mixer.rot_dim))
+    assert qa.shape == (n, mixer.num_q_heads * k_dim)
     assert freq.dtype == torch.float64 and freq.numel() == mixer.rot_dim // 2
     assert tok_pos.dtype == torch.int32 and tok_pos.shape[0] == n
     kp, vp, stride = _pool_ptrs(pool if dkv_col >= 0 else None, pool_slice)
@@ -59,8 +94,8 @@ def latent_rope_and_store_kv(proj: torch.Tensor, qa: torch.Tensor, freq: torch.T
     _hip.call("swl_latent_rope_store_kv", _hip.ptr(proj), _hip.ptr(qa), _hip.ptr(freq), _hip.ptr(c_norm), kp, vp,
               _hip.ptr(block_table), _hip.ptr(tok_seq), _hip.ptr(tok_pos), n, mixer.num_q_heads, mixer.head_dim,
               mixer.rot_dim, mixer.kv_rank, proj.stride(0), dkv_col if kp else -1, qa.stride(0),
-              block_table.shape[1] if block_table is not None else 0, stride, float(eps), _hip.dtype_code3(proj.dtype),
-              _hip.stream())
+              block_table.shape[1] if block_table is not None else 0, stride, float(eps), 1 if mixer.rot.half else 0,
+              float(mixer.rot.multiplier), k_dim, v_dim, _hip.dtype_code3(proj.dtype), _hip.stream())
 
 
 def diff_head_combine(maps: torch.Tensor, gate: torch.Tensor, lam: float, mult: float, eps: float, num_heads: int,

@@ -198,6 +198,28 @@ def masked_tiles_supported(spec: AttentionSpec, dtype: torch.dtype) -> bool:
                                                             spec.head_dim, spec.value_dim, _hip.dtype_code(dtype)))
 
 
+_row_sizes = {}     # (dim, vdim, dtype) -> served_row_sizes
+PADDING_LIMIT = 2.5
+
+
+def served_row_sizes(dim: int, vdim: int, dtype: torch.dtype):
+    """Key and value row sizes (in elements) that a layer with heads of `dim` / `vdim` should use in the pool: the smallest ones at
+    least as large that the matrix-core kernel is compiled for — rows are then padded with zeros, which change neither scores nor
+    outputs — or (dim, vdim) itself where padding would cost more than PADDING_LIMIT times the arithmetic, or in fp32."""
+    if dtype == torch.float32:
+        return dim, vdim
+    key = (dim, vdim, dtype)
+    if key not in _row_sizes:
+        best, lib, code = (dim, vdim), _hip.load(), _hip.dtype_code(dtype)
+        cost = PADDING_LIMIT * (dim + vdim)
+        for kd in range(-(-dim // 16) * 16, int(cost) + 1, 16):
+            for vd in range(-(-vdim // 16) * 16, int(cost) - kd + 1, 16):
+                if kd + vd < cost and lib.swl_masked_attn_tiles_supported(1, 1, 1, kd, vd, code):
+                    best, cost = (kd, vd), kd + vd
+        _row_sizes[key] = best
+    return _row_sizes[key]
+
+
 # From this many heads over one shared key head on, a step of single tokens runs with the heads on the matrix-core tile's rows
 HEAD_ROWS_MIN_HEADS = 2
 

@@ -10,12 +10,13 @@ from swiftllm_amd import _hip
 
 
 class StepContext:
-    """What the sublayers of one step share: the block pool and table, the per-token plan arrays, the state slots."""
-    __slots__ = ("pool", "block_table", "tok_seq", "tok_pos", "tiles", "state")
+    """What the sublayers of one step share: the block pool and table, the per-token plan arrays, the state slots, the portions'
+    chunks (chunk_row0, chunk_cnt, seq_chunk0: designs whose recurrence runs in parallel over them)."""
+    __slots__ = ("pool", "block_table", "tok_seq", "tok_pos", "tiles", "state", "chunks")
 
-    def __init__(self, pool, block_table, tok_seq, tok_pos, tiles, state):
-        self.pool, self.block_table, self.tok_seq, self.tok_pos, self.tiles, self.state = \
-            pool, block_table, tok_seq, tok_pos, tiles, state
+    def __init__(self, pool, block_table, tok_seq, tok_pos, tiles, state, chunks=None):
+        self.pool, self.block_table, self.tok_seq, self.tok_pos, self.tiles, self.state, self.chunks = \
+            pool, block_table, tok_seq, tok_pos, tiles, state, chunks
 
 
 class LorulixAttention:
@@ -68,7 +69,7 @@ class LorulixFeedForward:
         if mlp.kind == "dense":
             gu = _project(h, w.gate_up, self.skinny)
             y = torch.empty((h.shape[0], mlp.ffn_inter_dim), dtype=h.dtype, device=h.device)
-            _hip.call("swl_glu_clamp", _hip.ptr(y), _hip.ptr(gu), h.shape[0], mlp.ffn_inter_dim, float(mlp.limit), 0,
+            _hip.call("swl_glu_clamp", _hip.ptr(y), _hip.ptr(gu), 0, h.shape[0], mlp.ffn_inter_dim, float(mlp.limit), 0,
                       _hip.dtype_code3(h.dtype), _hip.stream())
             return _project(y, w.down, self.skinny), None, None
         idx, wts = moe_route_scores(h, w.router, mlp.top_k, mlp.router_scale)

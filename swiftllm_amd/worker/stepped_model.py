@@ -165,7 +165,7 @@ class SteppedModel:
     @torch.inference_mode()
     def step(self, entries: Sequence[StepEntry], ignore_kvcache: bool = False) -> torch.Tensor:
         """Run one batch of portions. Returns the logits of the wanted places, [wanted, vocab] (device tensor in the compute
-        dtype), in the order of the entries and of each entry's `want`."""
+        dtype; fp32 from a design that caps them), in the order of the entries and of each entry's `want`."""
         cfg = self.model_config
         plan = plan_step(entries, cfg.vocab_size, cfg.max_position_embeddings)
         if plan.num_tokens == 0:
