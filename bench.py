@@ -96,12 +96,12 @@ def parse_args():
     ap.add_argument("--no-reference", action="store_true", help="skip the reference-Triton child run")
     ap.add_argument("--compare-designs", action="store_true",
                     help="instead of the headline workload: prefill and decode throughput of the other designs (Kekapel, "
-                         "Lorulix, Rosilix, Ratilorn) beside LLaMA at equal layer sizes (random weights), one JSON line "
-                         "with all")
-    ap.add_argument("--compare", default="llama,kekapel,lorulix,rosilix,ratilorn",
+                         "Lorulix, Rosilix, Ratilorn, Rokevik) beside LLaMA at equal layer sizes (random weights), one "
+                         "JSON line with all")
+    ap.add_argument("--compare", default="llama,kekapel,lorulix,rosilix,ratilorn,rokevik",
                     help="designs that --compare-designs runs (comma list)")
     ap.add_argument("--compare-kv-rank", type=int, default=512,
-                    help="latent size of Rosilix's latent attention layers in --compare-designs")
+                    help="latent size of Rosilix's and Rokevik's latent attention layers in --compare-designs")
     ap.add_argument("--compare-sizes", default="small,medium", help="comma list out of " + ",".join(COMPARE_SIZES))
     return ap.parse_args()
 
@@ -178,7 +178,21 @@ def _compare_configs(sz, positions, kv_rank=512):
                     mlp=(tmoe if i % 2 else tdense)) for i in range(sz["layers"])]
     ratilorn = dict(architecture="Ratilorn", layers=tlayers, max_positions=positions, norm=dict(eps=1e-6), logit_scale=0.5,
                     vocab=sz["vocab"], width=sz["width"])
-    return llama, kekapel, lorulix, rosilix, ratilorn
+    # Rokevik at the same sizes: keys-as-values attention (rotary on half of each head) / two latent attentions (Rosilix's sizes,
+    # windows of 1024, interpolated rotary) / minGRU of the heads' total width, in turn; two streams, norms in two parts; every
+    # feed-forward a mixture of Ratilorn's sizes (8 experts of ff / 4, top 2, a shared one), no loop
+    kvattn = dict(dim=sz["dim"], vdim=sz["dim"], heads=sz["heads"], kv_heads=sz["kv_heads"], scale=sz["dim"] ** -0.5,
+                  softcap=50.0, rot=dict(base=10000.0, dims=half))
+    klat = dict(heads=sz["heads"], dim=sz["dim"], rot_dim=half, vdim=sz["dim"], kv_rank=kv_rank, mask=dict(size=1024),
+                rot=dict(base=500000.0, dims=half, scaling=dict(factor=8.0, original=1024, fast=32.0, slow=1.0)),
+                scale=(sz["dim"] + half) ** -0.5)
+    kmoe = dict(kind="moe", expert=dict(ff=sz["ff"] // 4), router=dict(experts=8, top=2), shared=dict(ff=sz["ff"] // 4))
+    kinds = (("attention", kvattn), ("latent_attention", klat), ("latent_attention", klat),
+             ("mingru", dict(width=sz["heads"] * sz["dim"])))
+    klayers = [dict(type=kinds[i % 4][0], mixer=dict(kinds[i % 4][1]), mlp=kmoe) for i in range(sz["layers"])]
+    rokevik = dict(architecture="Rokevik", layers=klayers, max_positions=positions, norm=dict(eps=1e-6, groups=2), streams=2,
+                   logit_softcap=30.0, vocab=sz["vocab"], width=sz["width"])
+    return llama, kekapel, lorulix, rosilix, ratilorn, rokevik
 
 
 def _compare_one(cfg, dtype, prompt_len, prompt_batch, decode_batch, decode_ctx, steps, warmup):
@@ -243,12 +257,13 @@ def run_compare_designs(args):
     Kekapel — the closest existing design: the same worker, stream and expert kernels — Lorulix / LLaMA, Rosilix over
     each of the three: Kekapel is its closest, an all-attention design on the same worker and attention kernels, and Ratilorn
     over Lorulix — its closest: attention beside a recurrence with state slots, experts with a shared one — Kekapel and
-    LLaMA)."""
+    LLaMA; Rokevik over Rosilix — its closest mixers: latent attention and rotary heads — Ratilorn — its closest feed-forwards and
+    state slots — Kekapel and LLaMA)."""
     results = {}
     for name in [s for s in args.compare_sizes.split(",") if s]:
         sz = COMPARE_SIZES[name]
         prompt_len, prompt_batch, decode_batch, decode_ctx = 2048, 4, 32, 1024
-        configs = dict(zip(("llama", "kekapel", "lorulix", "rosilix", "ratilorn"),
+        configs = dict(zip(("llama", "kekapel", "lorulix", "rosilix", "ratilorn", "rokevik"),
                            _compare_configs(sz, prompt_len + 256, args.compare_kv_rank)))
         rec = {"sizes": sz, "prompt": [prompt_batch, prompt_len], "decode": [decode_batch, decode_ctx]}
         for label in [d for d in args.compare.split(",") if d]:
@@ -259,7 +274,9 @@ def run_compare_designs(args):
                           ("lorulix", "llama", "lorulix_vs_llama_"), ("rosilix", "kekapel", "rosilix_vs_kekapel_"),
                           ("rosilix", "lorulix", "rosilix_vs_lorulix_"), ("rosilix", "llama", "rosilix_vs_llama_"),
                           ("ratilorn", "lorulix", "ratilorn_vs_lorulix_"), ("ratilorn", "kekapel", "ratilorn_vs_kekapel_"),
-                          ("ratilorn", "llama", "ratilorn_vs_llama_")):
+                          ("ratilorn", "llama", "ratilorn_vs_llama_"), ("rokevik", "rosilix", "rokevik_vs_rosilix_"),
+                          ("rokevik", "ratilorn", "rokevik_vs_ratilorn_"), ("rokevik", "kekapel", "rokevik_vs_kekapel_"),
+                          ("rokevik", "llama", "rokevik_vs_llama_")):
             if a in rec and b in rec:
                 rec[key + "prefill_ratio"] = rec[a]["prefill_tokens_per_s"] / rec[b]["prefill_tokens_per_s"]
                 rec[key + "decode_ratio"] = rec[a]["decode_tokens_per_s"] / rec[b]["decode_tokens_per_s"]
