@@ -628,7 +628,7 @@ int swl_moe_gate_up(void *y, const void *h, const void *gate_up, const int32_t *
  * multiplies it with all assignments of the expert (an expert's weights are streamed once per step). glu = 1: out = y[T * top, ff] from x = h[T, width]
  * and w = gate_up; glu = 0: out = rows[T * top, width] (plain products, for swl_moe_combine) from x = y and w = down.
  * act (swl_moe_gate_up, swl_glu_clamp): 0 the clamped unit min(g, limit) sigmoid(1.702 g) (clamp(u) + 1), 1 the plain gated
- * unit silu(g) u (limit unused); swl_moe_expert_stationary takes the latter as glu = 3. in_w (NULL: none): a weight per
+ * unit silu(g) u (limit unused), swl_glu_clamp also 2: the latter on rows [up | gate]; swl_moe_expert_stationary takes it as glu = 3. in_w (NULL: none): a weight per
  * assignment (swl_glu_clamp: per row) on the expert's input, applied to the fp32 products g and u. expert_w of the two
  * combinations may be NULL (all one). */
 int swl_moe_expert_stationary_supported(int64_t num_tokens, int32_t width, int32_t ff, int32_t top, int32_t dtype);
@@ -779,14 +779,14 @@ int swl_qk_norm_rope_store_kv(const void *rows, void *q_out, const float *q_b, c
 
 /* ---- fp32 residual of several streams, hyper-connections (csrc/hyper_stream.hip) ------------------------------------------------
  * x [rows, streams, width] fp32. swl_embed_streams: every stream = embed[token]. swl_hyper_step: with y (+ y2, + y_bias[width])
- * the previous sublayer's result, X_t <- sum_s mix[s][t] X_s + outw[t] y (all from the old streams); then, with h given,
+ * the previous sublayer's result (the fp32 sum of y_parts rows y[t * y_parts + j]), X_t <- sum_s mix[s][t] X_s + outw[t] y (all from the old streams); then, with h given,
  * u = sum_s inw[s] X_s (inw NULL: plain sum) and h = u / rms(u in `groups` equal parts; eps) * norm_w. y NULL: norm only, of
- * rows row_idx when given; h NULL: update only. At most 8 streams. dtype (y, y2, h) may be SWL_F32. */
+ * rows row_idx when given; h NULL: update only. At most 16 streams. dtype (y, y2, h) may be SWL_F32. */
 int swl_embed_streams(float *x, const void *embed, const int32_t *tokens, int64_t num_tokens, int32_t width, int32_t streams,
                       int32_t dtype, swl_stream_t stream);
-int swl_hyper_step(float *x, const void *y, const void *y2, const float *y_bias, const float *mix, const float *outw,
-                   const float *inw, const float *norm_w, void *h, const int32_t *row_idx, int64_t num_rows, int32_t width,
-                   int32_t streams, int32_t groups, float eps, int32_t dtype, swl_stream_t stream);
+int swl_hyper_step(float *x, const void *y, int32_t y_parts, const void *y2, const float *y_bias, const float *mix,
+                   const float *outw, const float *inw, const float *norm_w, void *h, const int32_t *row_idx, int64_t num_rows,
+                   int32_t width, int32_t streams, int32_t groups, float eps, int32_t dtype, swl_stream_t stream);
 
 /* ---- minGRU (csrc/min_gru.hip) -----------------------------------------------------------------------------------------------------
  * proj rows [z | u | gate] of width columns each; per channel a = sigmoid(z + z_b), c = u' + 1/2 (u' = u + u_b >= 0) or sigmoid(u'),

@@ -145,7 +145,7 @@ SIGNATURES = {
     "swl_qk_norm_rope_store_kv": [_P, _P, _P, _P, _P, _P, _P, _P, _P, _P, _P, _P, _P, _I64, _I32, _I32, _I32, _I32, _I32, _I32,
                                   _I32, _F64, _I64, _I64, _I32, _I32, _I32, _I32, _I64, _F32, _I32, _P],
     "swl_embed_streams": [_P, _P, _P, _I64, _I32, _I32, _I32, _P],
-    "swl_hyper_step": [_P, _P, _P, _P, _P, _P, _P, _P, _P, _P, _I64, _I32, _I32, _I32, _F32, _I32, _P],
+    "swl_hyper_step": [_P, _P, _I32, _P, _P, _P, _P, _P, _P, _P, _P, _I64, _I32, _I32, _I32, _F32, _I32, _P],
     "swl_min_gru_chunks": [_P, _P, _I64, _P, _P, _P, _P, _I32, _I32, _I32, _P],
     "swl_min_gru_carry": [_P, _P, _I64, _I64, _P, _P, _P, _P, _P, _I32, _I32, _I32, _P],
     "swl_min_gru_apply": [_P, _P, _I64, _P, _P, _P, _P, _I64, _I64, _P, _P, _P, _P, _I32, _I32, _I32, _P],

@@ -2,7 +2,8 @@
 //
 //   swl_embed_streams: x[t][s] = embed[token[t]] for every stream s.
 //   swl_hyper_step:    the step between two sublayers in one launch, one workgroup per token. With the previous sublayer's result
-//                      y (+ y2: a second addend, + y_bias: a bias of its output projection)
+//                      y (the sum of y_parts rows per token: the results of a token's experts; + y2: a second addend, + y_bias: a
+//                      bias of its output projection)
 //       X_t <- sum_s mix[s][t] X_s + out[t] * y        all streams at once from the old ones
 //       u    = sum_s in[s] X_s                         what the next sublayer reads
 //       h    = u / rms(u over each of `groups` equal parts) * w
@@ -16,7 +17,7 @@
 namespace swl {
 
 constexpr int kHsThreads = 256;
-constexpr int kHsMaxStreams = 8;
+constexpr int kHsMaxStreams = 16;
 constexpr int kHsQuickGroups = 4;       // norm parts whose sums are kept in registers
 
 template <typename T>
@@ -56,7 +57,7 @@ __device__ __forceinline__ void hs_store(T *p, const float *src) {
 // S: streams held in registers (S == streams when EXACT, else S >= streams). V: columns per access (4 when width % 4 == 0).
 template <typename T, int S, int V, bool EXACT>
 __global__ __launch_bounds__(kHsThreads) void hyper_step_kernel(
-    float *x, const T *y, const T *y2, const float *y_bias, const float *__restrict__ mix, const float *__restrict__ outw,
+    float *x, const T *y, int y_parts, const T *y2, const float *y_bias, const float *__restrict__ mix, const float *__restrict__ outw,
     const float *__restrict__ inw, const float *__restrict__ norm_w, T *h, const int32_t *row_idx, int width, int streams,
     int groups, float eps) {
     extern __shared__ float lds[];
@@ -88,7 +89,13 @@ __global__ __launch_bounds__(kHsThreads) void hyper_step_kernel(
         for (int j = 0; j < V; ++j) u[j] = 0.f;
         if (y) {
             float yv[V];
-            hs_load<T, V>(yv, y + t * width + c);
+            hs_load<T, V>(yv, y + t * y_parts * width + c);
+            for (int k = 1; k < y_parts; ++k) {
+                float b[V];
+                hs_load<T, V>(b, y + (t * y_parts + k) * width + c);
+#pragma unroll
+                for (int j = 0; j < V; ++j) yv[j] += b[j];
+            }
             if (y2) {
                 float b[V];
                 hs_load<T, V>(b, y2 + t * width + c);
@@ -188,18 +195,21 @@ inline size_t hs_lds_bytes(int width, int groups) {
 }
 
 template <typename T, int V>
-void launch_hs(dim3 grid, size_t lds, hipStream_t s, float *x, const T *y, const T *y2, const float *yb, const float *mix,
+void launch_hs(dim3 grid, size_t lds, hipStream_t s, float *x, const T *y, int yp, const T *y2, const float *yb, const float *mix,
                const float *ow, const float *iw, const float *nw, T *h, const int32_t *ri, int width, int streams, int groups,
                float eps) {
 #define SWL_HS(S, X)                                                                                                          \
-    hipLaunchKernelGGL((hyper_step_kernel<T, S, V, X>), grid, dim3(kHsThreads), lds, s, x, y, y2, yb, mix, ow, iw, nw, h, ri, \
+    hipLaunchKernelGGL((hyper_step_kernel<T, S, V, X>), grid, dim3(kHsThreads), lds, s, x, y, yp, y2, yb, mix, ow, iw, nw, h, ri, \
                        width, streams, groups, eps)
     switch (streams) {
     case 1: SWL_HS(1, true); break;
     case 2: SWL_HS(2, true); break;
     case 3: SWL_HS(3, true); break;
     case 4: SWL_HS(4, true); break;
-    default: SWL_HS(kHsMaxStreams, false); break;
+    default:
+        if (streams <= 8) SWL_HS(8, false);
+        else SWL_HS(kHsMaxStreams, false);
+        break;
     }
 #undef SWL_HS
 }
@@ -219,9 +229,11 @@ extern "C" int swl_embed_streams(float *x, const void *embed, const int32_t *tok
     return swl::check_launch();
 }
 
-extern "C" int swl_hyper_step(float *x, const void *y, const void *y2, const float *y_bias, const float *mix, const float *outw,
-                              const float *inw, const float *norm_w, void *h, const int32_t *row_idx, int64_t num_rows,
-                              int32_t width, int32_t streams, int32_t groups, float eps, int32_t dtype, swl_stream_t stream) {
+extern "C" int swl_hyper_step(float *x, const void *y, int32_t y_parts, const void *y2, const float *y_bias, const float *mix,
+                              const float *outw, const float *inw, const float *norm_w, void *h, const int32_t *row_idx,
+                              int64_t num_rows, int32_t width, int32_t streams, int32_t groups, float eps, int32_t dtype,
+                              swl_stream_t stream) {
+    if (y && y_parts < 1) return SWL_ERR_BAD_ARG;
     if (num_rows < 0 || width <= 0 || streams <= 0 || groups <= 0 || width % groups) return SWL_ERR_BAD_ARG;
     if (num_rows == 0) return SWL_OK;
     if (!x || (y && (!mix || !outw)) || (!y && (y2 || y_bias)) || (h && !norm_w) || (row_idx && y)) return SWL_ERR_BAD_ARG;
@@ -234,10 +246,10 @@ extern "C" int swl_hyper_step(float *x, const void *y, const void *y2, const flo
     hipStream_t s = static_cast<hipStream_t>(stream);
     SWL_DISPATCH_DTYPE3(dtype, T, {
         if (wide)
-            swl::launch_hs<T, 4>(grid, lds, s, x, static_cast<const T *>(y), static_cast<const T *>(y2), y_bias, mix, outw, inw,
+            swl::launch_hs<T, 4>(grid, lds, s, x, static_cast<const T *>(y), y_parts, static_cast<const T *>(y2), y_bias, mix, outw, inw,
                                  norm_w, static_cast<T *>(h), row_idx, width, streams, groups, eps);
         else
-            swl::launch_hs<T, 1>(grid, lds, s, x, static_cast<const T *>(y), static_cast<const T *>(y2), y_bias, mix, outw, inw,
+            swl::launch_hs<T, 1>(grid, lds, s, x, static_cast<const T *>(y), y_parts, static_cast<const T *>(y2), y_bias, mix, outw, inw,
                                  norm_w, static_cast<T *>(h), row_idx, width, streams, groups, eps);
     });
     return swl::check_launch();

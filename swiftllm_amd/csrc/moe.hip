@@ -15,7 +15,7 @@
 //                         products are linear, so it multiplies their fp32 sums: act(w g, w u). The combination then takes no
 //                         weights (NULL: all one).
 //   act (swl_moe_gate_up, swl_glu_clamp; glu = 3 of swl_moe_expert_stationary): 0 the clamped unit above, 1 the plain gated
-//                         unit y = silu(g) * u.
+//                         unit y = silu(g) * u, 2 (swl_glu_clamp only) the same on rows [up | gate].
 //
 // Expert weights are stacked: gate_up [experts, 2 ff, width] (gate rows, then up rows), down [experts, width, ff].
 #include "swl_common.h"
@@ -63,9 +63,10 @@ __device__ __forceinline__ float lane_dot2(const T *x, const T *w, int n, int la
     return a;
 }
 
-// act 0: g' = min(g, limit), u' = clamp(u, +-limit), g' sigmoid(1.702 g') (u' + 1); act 1: silu(g) u
+// act 0: g' = min(g, limit), u' = clamp(u, +-limit), g' sigmoid(1.702 g') (u' + 1); act 1: silu(g) u; act 2: silu(u) g
 __device__ __forceinline__ float gated_unit(float g, float u, float limit, int act) {
     if (act == 1) return g / (1.0f + expf(-g)) * u;
+    if (act == 2) return u / (1.0f + expf(-u)) * g;
     g = fminf(g, limit);
     u = fminf(fmaxf(u, -limit), limit);
     return g * (1.0f / (1.0f + expf(-1.702f * g))) * (u + 1.0f);
@@ -590,7 +591,7 @@ extern "C" int swl_moe_expert_stationary(void *out, const void *x, const void *w
 
 extern "C" int swl_glu_clamp(void *y, const void *gate_up, const float *in_w, int64_t num_rows, int32_t ff, float limit,
                              int32_t act, int32_t dtype, swl_stream_t stream) {
-    if (num_rows < 0 || ff <= 0 || act < 0 || act > 1) return SWL_ERR_BAD_ARG;
+    if (num_rows < 0 || ff <= 0 || act < 0 || act > 2) return SWL_ERR_BAD_ARG;
     if (num_rows == 0) return SWL_OK;
     if (!y || !gate_up) return SWL_ERR_BAD_ARG;
     const bool wide = dtype != SWL_F32 && ff % 8 == 0 && swl::aligned16(y) && swl::aligned16(gate_up);

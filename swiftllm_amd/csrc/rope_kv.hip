@@ -98,8 +98,6 @@ __global__ __launch_bounds__(kRkThreads) void qk_norm_rope_store_kv_kernel(
     const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
     const int pos = tok_pos[t];
     const int pairs = rot_dims >> 1;
-    rk_angles(cs, sn, freq, pos, pairs, rot_mult);
-    __syncthreads();
     const T *row = rows + t * tok_stride;
     T *qrow = q_out + t * q_out_stride;
     const bool store = k_cache != nullptr;
@@ -121,36 +119,63 @@ __global__ __launch_bounds__(kRkThreads) void qk_norm_rope_store_kv_kernel(
             const int lph = d <= 8 ? 1 : d <= 16 ? 2 : d <= 32 ? 4 : d <= 64 ? 8 : 16;      // lanes per head
             const int hpw = 64 / lph;
             const int slot = lane / lph, el = lane - slot * lph, e0 = el * 8;
-            auto load_biased = [&](float *v, const T *p, const float *b) {
-                const vec8_t<T> x = load8(p);
-#pragma unroll
-                for (int j = 0; j < 8; ++j) v[j] = to_f(x[j]);
-                if (b) {
-                    const float4_t b0 = *reinterpret_cast<const float4_t *>(b), b1 = *reinterpret_cast<const float4_t *>(b + 4);
-#pragma unroll
-                    for (int j = 0; j < 4; ++j) {
-                        v[j] += b0[j];
-                        v[4 + j] += b1[j];
-                    }
-                }
-            };
-            for (int hb = wave * hpw; hb < heads; hb += (kRkThreads / 64) * hpw) {
+            const bool turns = e0 < rot_dims, first = e0 < pairs;
+            // (half) the partner elements of this lane's, and the pair index of its first element
+            const int p0 = half && turns ? (first ? e0 + pairs : e0 - pairs) : e0;
+            const int a0 = half ? (first ? e0 : p0) : e0 >> 1;
+            // everything a head needs from memory is requested together, the first head's before the angles are evaluated
+            vec8_t<T> own, other;
+            float4_t bo[2], bp[2], wo[2], wp[2];
+            float mult;
+            auto fetch = [&](int hb) {
                 const int h = hb + slot;
                 const bool live = h < heads && e0 < d, is_q = h < nq;
-                const T *src = row + static_cast<int64_t>(live ? h : 0) * d;
+                own = other = vec8_t<T>{};
+                mult = 1.0f;
+#pragma unroll
+                for (int k = 0; k < 2; ++k) {
+                    bo[k] = bp[k] = float4_t{0.f, 0.f, 0.f, 0.f};
+                    wo[k] = wp[k] = float4_t{1.f, 1.f, 1.f, 1.f};
+                }
+                if (!live) return;
+                const T *src = row + static_cast<int64_t>(h) * d;
                 const float *bias = is_q ? q_b : k_b, *wn = is_q ? q_w : k_w;
-                if (bias) bias += static_cast<int64_t>(live ? (is_q ? h : h - nq) : 0) * d;
+                own = load8(src + e0);
+                other = load8(src + p0);
+                if (bias) {
+                    bias += static_cast<int64_t>(is_q ? h : h - nq) * d;
+#pragma unroll
+                    for (int k = 0; k < 2; ++k) {
+                        bo[k] = *reinterpret_cast<const float4_t *>(bias + e0 + 4 * k);
+                        bp[k] = *reinterpret_cast<const float4_t *>(bias + p0 + 4 * k);
+                    }
+                }
+                if (wn) {
+#pragma unroll
+                    for (int k = 0; k < 2; ++k) {
+                        wo[k] = *reinterpret_cast<const float4_t *>(wn + e0 + 4 * k);
+                        wp[k] = *reinterpret_cast<const float4_t *>(wn + p0 + 4 * k);
+                    }
+                }
+                if (is_q && q_mult) mult = q_mult[h];
+            };
+            fetch(wave * hpw);
+            rk_angles(cs, sn, freq, pos, pairs, rot_mult);
+            __syncthreads();
+            for (int hb = wave * hpw; hb < heads; hb += (kRkThreads / 64) * hpw) {
+                if (hb != wave * hpw) fetch(hb);
+                const int h = hb + slot;
+                const bool live = h < heads && e0 < d, is_q = h < nq;
                 float v[8];
 #pragma unroll
-                for (int j = 0; j < 8; ++j) v[j] = 0.f;
-                if (live) load_biased(v, src + e0, bias ? bias + e0 : nullptr);
+                for (int j = 0; j < 8; ++j) v[j] = to_f(own[j]) + bo[j >> 2][j & 3];
                 float ss = 0.f;
 #pragma unroll
                 for (int j = 0; j < 8; ++j) ss += v[j] * v[j];
                 ss = lph == 1 ? ss : lph == 2 ? group_allreduce_sum<2>(ss) : lph == 4 ? group_allreduce_sum<4>(ss)
                    : lph == 8 ? group_allreduce_sum<8>(ss) : group_allreduce_sum<16>(ss);
-                const float r = wn ? 1.0f / sqrtf(ss / static_cast<float>(d) + eps) : 1.0f;
                 if (!live) continue;
+                const float r = (is_q ? q_w : k_w) ? 1.0f / sqrtf(ss / static_cast<float>(d) + eps) : 1.0f;
                 if (!is_q && keys_as_values) {
                     T *dst = vpage + (static_cast<int64_t>(h - nq) * v_dim + e0) * kRkBlock + off;
 #pragma unroll
@@ -158,28 +183,21 @@ __global__ __launch_bounds__(kRkThreads) void qk_norm_rope_store_kv_kernel(
                 }
                 float n[8];
 #pragma unroll
-                for (int j = 0; j < 8; ++j) n[j] = wn ? v[j] * r * wn[e0 + j] : v[j];
-                if (e0 < rot_dims) {
-                    if (half) {
-                        const bool first = e0 < pairs;
-                        const int p0 = first ? e0 + pairs : e0 - pairs, a0 = first ? e0 : p0;
-                        float o[8];
-                        load_biased(o, src + p0, bias ? bias + p0 : nullptr);
+                for (int j = 0; j < 8; ++j) n[j] = v[j] * r * wo[j >> 2][j & 3];
+                if (turns && half) {
 #pragma unroll
-                        for (int j = 0; j < 8; ++j) {
-                            const float w = wn ? o[j] * r * wn[p0 + j] : o[j];
-                            n[j] = first ? n[j] * cs[a0 + j] - w * sn[a0 + j] : n[j] * cs[a0 + j] + w * sn[a0 + j];
-                        }
-                    } else {
+                    for (int j = 0; j < 8; ++j) {
+                        const float w = (to_f(other[j]) + bp[j >> 2][j & 3]) * r * wp[j >> 2][j & 3];
+                        n[j] = first ? n[j] * cs[a0 + j] - w * sn[a0 + j] : n[j] * cs[a0 + j] + w * sn[a0 + j];
+                    }
+                } else if (turns) {
 #pragma unroll
-                        for (int j = 0; j < 8; j += 2) {
-                            const float c = cs[(e0 + j) >> 1], sv = sn[(e0 + j) >> 1], u = n[j], w = n[j + 1];
-                            n[j] = u * c - w * sv;
-                            n[j + 1] = w * c + u * sv;
-                        }
+                    for (int j = 0; j < 8; j += 2) {
+                        const float c = cs[a0 + (j >> 1)], sv = sn[a0 + (j >> 1)], u = n[j], w = n[j + 1];
+                        n[j] = u * c - w * sv;
+                        n[j + 1] = w * c + u * sv;
                     }
                 }
-                const float mult = is_q && q_mult ? q_mult[h] : 1.0f;
                 vec8_t<T> o;
 #pragma unroll
                 for (int j = 0; j < 8; ++j) o[j] = to_t<T>(n[j] * mult);
@@ -187,6 +205,10 @@ __global__ __launch_bounds__(kRkThreads) void qk_norm_rope_store_kv_kernel(
                             : kpage + (static_cast<int64_t>(h - nq) * kRkBlock + off) * k_dim + e0, o);
             }
         }
+    }
+    if (!wide) {
+        rk_angles(cs, sn, freq, pos, pairs, rot_mult);
+        __syncthreads();
     }
     for (int h = wave; h < heads && !wide; h += kRkThreads / 64) {
         const bool is_q = h < nq;

@@ -815,6 +815,7 @@ class RokevikModelConfig:
     config.json. `streams` absent: one plain residual. The design has no position table: `max_positions`, if config.json gives
     it, bounds a sequence; otherwise the bound is DEFAULT_MAX_POSITIONS."""
     DEFAULT_MAX_POSITIONS = 1 << 20
+    MAX_STREAMS = 16            # (what the streams' kernel holds in registers: csrc/hyper_stream.hip)
 
     def __init__(self, model_config: dict):
         if model_config.get("architecture") != "Rokevik":
@@ -827,6 +828,8 @@ class RokevikModelConfig:
         if self.norm_groups < 1 or self.hidden_size % self.norm_groups:
             raise ValueError(f"width ({self.hidden_size}) must be a multiple of norm.groups ({self.norm_groups})")
         self.num_streams = int(model_config.get("streams") or 0)        # 0: a plain residual, no stream weights
+        if not 0 <= self.num_streams <= self.MAX_STREAMS:
+            raise ValueError(f"streams ({self.num_streams}) must be at most {self.MAX_STREAMS}")
         cap = model_config.get("logit_softcap")
         self.logit_softcap = float(cap) if cap else 0.0
         self.layers = [RokevikLayerConfig(layer) for layer in model_config["layers"]]

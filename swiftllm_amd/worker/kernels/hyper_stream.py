@@ -36,7 +36,8 @@ def hyper_step(x: torch.Tensor, y: torch.Tensor = None, done: StreamWeights = No
                y_bias: torch.Tensor = None, read: torch.Tensor = None, norm: torch.Tensor = None, groups: int = 1,
                eps: float = 1e-6, out_dtype: torch.dtype = None, row_idx: torch.Tensor = None) -> torch.Tensor:
     """The step between two sublayers on the streams x [T, S, width], in place. y (+ y2, + y_bias [width] fp32): the result of the
-    sublayer whose StreamWeights are `done`. norm (fp32 [width]): returns the next input, the sum of the streams weighted by
+    sublayer whose StreamWeights are `done`; y has one row per token, or k neighbouring ones (the results of its k experts) that
+    are summed. norm (fp32 [width]): returns the next input, the sum of the streams weighted by
     `read` (None: plainly summed), RMS-normed in `groups` equal parts and scaled by `norm`, in y's dtype (out_dtype without a y) —
     of rows row_idx only, when given; then y must be None."""
     _hip.require_gpu_tensor(x, "x")
@@ -44,14 +45,14 @@ def hyper_step(x: torch.Tensor, y: torch.Tensor = None, done: StreamWeights = No
     assert x.dtype == torch.float32 and x.is_contiguous() and (y is not None or norm is not None)
     dtype = y.dtype if y is not None else out_dtype
     if y is not None:
-        assert y.shape == (n, width) and y.is_contiguous() and done.mix.shape[0] == streams
-        assert y2 is None or (y2.shape == y.shape and y2.is_contiguous() and y2.dtype == y.dtype)
+        assert y.shape[1] == width and y.shape[0] % n == 0 and y.is_contiguous() and done.mix.shape[0] == streams
+        assert y2 is None or (y2.shape == (n, width) and y2.is_contiguous() and y2.dtype == y.dtype)
     assert read is None or (read.dtype == torch.float32 and read.numel() == streams)
     for w in (y_bias, norm):
         assert w is None or (w.dtype == torch.float32 and w.is_contiguous() and w.numel() == width)
     rows = n if row_idx is None else row_idx.shape[0]
     out = torch.empty((rows, width), dtype=dtype, device=x.device) if norm is not None else None
-    _hip.call("swl_hyper_step", _hip.ptr(x), _hip.ptr(y), _hip.ptr(y2), _hip.ptr(y_bias),
+    _hip.call("swl_hyper_step", _hip.ptr(x), _hip.ptr(y), y.shape[0] // n if y is not None else 0, _hip.ptr(y2), _hip.ptr(y_bias),
               _hip.ptr(done.mix) if y is not None else 0, _hip.ptr(done.write) if y is not None else 0, _hip.ptr(read),
               _hip.ptr(norm), _hip.ptr(out), _hip.ptr(row_idx), rows, width, streams, int(groups), float(eps),
               _hip.dtype_code3(dtype), _hip.stream())

@@ -111,6 +111,7 @@ def _identity(n: int, device) -> torch.Tensor:
 
 ACT_CLAMPED = 0     # min(g, limit) * sigmoid(1.702 g) * (clamp(u, +-limit) + 1)
 ACT_SILU = 1        # silu(g) * u
+ACT_SILU_UP_FIRST = 2       # the same on rows [up | gate] (gated_unit only)
 
 
 def gated_unit(gu: torch.Tensor, ff: int, act: int = ACT_SILU, limit: float = 0.0, in_w: torch.Tensor = None) -> torch.Tensor:
@@ -177,11 +178,12 @@ def moe_experts_grouped(h: torch.Tensor, idx: torch.Tensor, wts: torch.Tensor, g
 
 
 def moe_experts(h: torch.Tensor, idx: torch.Tensor, wts: torch.Tensor, gate_up: torch.Tensor, down: torch.Tensor,
-                limit: float, act: int = ACT_CLAMPED, weigh_inputs: bool = False) -> torch.Tensor:
+                limit: float, act: int = ACT_CLAMPED, weigh_inputs: bool = False, combine: bool = True) -> torch.Tensor:
     """-> [T, width]: sum_j wts[t, j] * expert idx[t, j] applied to h[t]. gate_up [experts, 2 ff, width], down
     [experts, width, ff]. act: the experts' gated unit (ACT_CLAMPED with `limit`, or ACT_SILU). weigh_inputs: the weights
     multiply the experts' inputs instead, sum_j expert(wts[t, j] * h[t]) — applied to the fp32 products of the gate and up rows
-    (to their rounded products in the sorted form), which are linear in the input."""
+    (to their rounded products in the sorted form), which are linear in the input. combine False (with weigh_inputs): a step that
+    has the experts' results as rows [T * top_k, width] hands them over un-summed (the caller's next step adds them)."""
     n, width = h.shape
     experts, two_ff, _ = gate_up.shape
     ff, top_k = two_ff // 2, idx.shape[1]
@@ -199,6 +201,8 @@ def moe_experts(h: torch.Tensor, idx: torch.Tensor, wts: torch.Tensor, gate_up: 
         rows = torch.empty((n * top_k, width), dtype=h.dtype, device=h.device)
         _hip.call("swl_moe_expert_stationary", _hip.ptr(rows), _hip.ptr(y), _hip.ptr(down), _hip.ptr(idx), 0, n, experts,
                   width, ff, top_k, 0, float(limit), code, stream)
+        if weigh_inputs and not combine:
+            return rows
         out = torch.empty((n, width), dtype=h.dtype, device=h.device)
         _hip.call("swl_moe_combine", _hip.ptr(out), _hip.ptr(rows), _hip.ptr(_identity(n * top_k, h.device)),
                   out_w, n, width, top_k, code, stream)

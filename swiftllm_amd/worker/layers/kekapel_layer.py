@@ -4,8 +4,8 @@ import torch
 
 from swiftllm_amd import _hip
 
-from ..kernels.linear import linear
-from ..kernels.moe import moe_experts, moe_route
+from ..kernels.linear import linear, linear_silu_gate
+from ..kernels.moe import ACT_SILU_UP_FIRST, gated_unit, moe_experts, moe_route
 from ..kernels.polynorm import polynorm
 from ..kernels.window_attn import qknorm_and_store_kv, window_attention
 
@@ -25,6 +25,21 @@ def _project(a: torch.Tensor, w: torch.Tensor, skinny: bool) -> torch.Tensor:
                 raise
             w._swl_blas_only = True
     return linear(a, w, False)
+
+
+def _silu_unit(a: torch.Tensor, up_gate: torch.Tensor, skinny: bool) -> torch.Tensor:
+    """(up a) * silu(gate a) for the stacked matrix [up; gate] -> [T, ff]: one launch for decode-sized 16-bit batches (the
+    product's epilogue), projection and activation otherwise."""
+    if skinny and a.dtype != torch.float32 and not getattr(up_gate, "_swl_no_silu", False):
+        try:
+            y = linear_silu_gate(a, up_gate)
+            if y is not None:
+                return y
+        except _hip.HipLibraryError as exc:
+            if "code -2" not in str(exc):       # (see _project)
+                raise
+            up_gate._swl_no_silu = True
+    return gated_unit(_project(a, up_gate, skinny), up_gate.shape[0] // 2, ACT_SILU_UP_FIRST)
 
 
 class KekapelAttention:

@@ -3,10 +3,10 @@ mixing the result into the streams and the next input's norm are the model's fus
 import torch
 
 from ..kernels.min_gru import min_gru
-from ..kernels.moe import ACT_SILU, gated_unit, moe_experts, moe_route_grouped
+from ..kernels.moe import ACT_SILU, moe_experts, moe_route_grouped
 from ..kernels.rope_kv import head_gate_, latent_rope_and_store_kv, qk_norm_rope_and_store_kv
 from ..kernels.window_attn import MASK_WINDOW, AttentionSpec, masked_attention
-from .kekapel_layer import _project
+from .kekapel_layer import _project, _silu_unit
 from .lorulix_layer import StepContext
 
 
@@ -89,8 +89,8 @@ class RokevikMinGru:
 
 
 class RokevikFeedForward:
-    """Sigmoid router -> SiLU gated experts on inputs scaled by their scores; the shared expert's result leaves separately (the
-    stream step adds the two)."""
+    """Sigmoid router -> SiLU gated experts on inputs scaled by their scores; the experts' results of decode-sized steps and the
+    shared expert's leave separately (the stream step adds them up)."""
 
     def __init__(self, layer_config, weight, skinny: bool):
         self.mlp, self.w, self.skinny = layer_config.mlp, weight, skinny
@@ -99,8 +99,7 @@ class RokevikFeedForward:
     def forward(self, h: torch.Tensor, ctx: StepContext):
         mlp, w = self.mlp, self.w
         idx, wts = moe_route_grouped(h, w.router, None, mlp.top_k, normalize=False)
-        out = moe_experts(h, idx, wts, w.gate_up, w.down, 0.0, ACT_SILU, weigh_inputs=True)
-        if w.shared_gate_up is None:
+        out = moe_experts(h, idx, wts, w.gate_up, w.down, 0.0, ACT_SILU, weigh_inputs=True, combine=False)
+        if w.shared_up_gate is None:
             return out, None
-        unit = gated_unit(_project(h, w.shared_gate_up, self.skinny), mlp.shared_ffn_inter_dim, ACT_SILU)
-        return out, _project(unit, w.shared_down, self.skinny)
+        return out, _project(_silu_unit(h, w.shared_up_gate, self.skinny), w.shared_down, self.skinny)

@@ -6,7 +6,8 @@ feed-forward's `mlp.*` and the stream weights `hc1.* / hc2.*` (`in`, `out`, `mix
 What the loader does with them:
   * matrices that multiply the same input are concatenated into one projection, padded with zero rows to a multiple of 8 rows so
     that every row of its output starts on a 16-byte boundary: attention q | k | head gate; latent attention q | compressed kv |
-    head gate; minGRU z | x | gate; feed-forwards gate | up, experts stacked ([experts, 2 ff, width], [experts, width, ff]);
+    head gate; minGRU z | x | gate; experts gate | up, stacked ([experts, 2 ff, width], [experts, width, ff]); the shared expert up | gate (the
+    order of the decode GEMM that applies the gate itself);
   * the latent attention's up-projections are kept per head for batched products: uk [H, dim, kv_rank] (queries are folded
     through it) and uv^T [H, kv_rank, vdim] (applied to the attention's output over the latent rows);
   * everything that enters fp32 arithmetic — norm weights, biases, head temperatures, the router, the stream weights — is kept in
@@ -83,10 +84,10 @@ class RokevikLayerWeight:
             self.gate_up[e, :ff] = mat(f"mlp.e{e}.gate", (ff, w))
             self.gate_up[e, ff:] = mat(f"mlp.e{e}.up", (ff, w))
             self.down[e] = mat(f"mlp.e{e}.down", (w, ff))
-        self.shared_gate_up = self.shared_down = None
+        self.shared_up_gate = self.shared_down = None
         if mlp.shared_ffn_inter_dim:
             fs = mlp.shared_ffn_inter_dim
-            self.shared_gate_up = torch.cat((mat("mlp.shared.gate", (fs, w)), mat("mlp.shared.up", (fs, w))), dim=0).contiguous()
+            self.shared_up_gate = torch.cat((mat("mlp.shared.up", (fs, w)), mat("mlp.shared.gate", (fs, w))), dim=0).contiguous()
             self.shared_down = mat("mlp.shared.down", (w, fs))
 
 
@@ -109,7 +110,7 @@ class RokevikWeight:
         """The 2-D matrices a step multiplies through `linear` (candidates for the decode GEMMs' packed copies)."""
         out = [self.head]
         for layer in self.layers:
-            for a in ("proj", "o", "shared_gate_up", "shared_down"):
+            for a in ("proj", "o", "shared_up_gate", "shared_down"):
                 t = getattr(layer, a, None)
                 if t is not None:
                     out.append(t)

@@ -78,7 +78,8 @@ def run_in_portions(model, seq, toks, sizes):
 
 # ---- the streams -------------------------------------------------------------------------------------------------------------
 @pytest.mark.parametrize("S,width,groups,n", [(1, 48, 1, 5), (2, 192, 2, 9), (3, 50, 5, 4), (4, 1024, 4, 7), (2, 36, 6, 3),
-                                              (5, 40, 1, 3), (8, 2052, 3, 4), (3, 33, 3, 6), (2, 4096, 1, 2), (4, 4100, 10, 2)])
+                                              (5, 40, 1, 3), (8, 2052, 3, 4), (3, 33, 3, 6), (2, 4096, 1, 2), (4, 4100, 10, 2),
+                                              (13, 44, 2, 3)])
 @pytest.mark.parametrize("dtype", [torch.float32, torch.bfloat16, torch.float16])
 def test_streams_step(S, width, groups, n, dtype):
     from swiftllm_amd.worker.kernels.hyper_stream import StreamWeights, embed_streams, hyper_step
@@ -104,6 +105,12 @@ def test_streams_step(S, width, groups, n, dtype):
         x2 = X.cuda().clone()
         assert hyper_step(x2, y.cuda(), sw, y2.cuda() if second else None, bias.cuda() if with_bias else None) is None
         assert torch.equal(x2, x)
+    # a result in three rows per token (a token's experts), summed
+    y3 = torch.randn(n, 3, width, generator=g).to(dtype)
+    new = O.hyper_step(Xs, d(y3).sum(1) + d(y2), d(mix), d(out))
+    x = X.cuda().clone()
+    hyper_step(x, y3.view(n * 3, width).cuda(), sw, y2.cuda())
+    assert (x.cpu().double() - new.transpose(0, 1)).abs().max() < 1e-5 * float(new.abs().max())
     # the norm alone: of all rows with a weighted sum, of some rows of the plain sum (the model's last norm); nothing is written
     x = X.cuda().clone()
     h = hyper_step(x, read=read.cuda(), norm=w.cuda(), groups=groups, eps=EPS, out_dtype=dtype)
@@ -484,7 +491,7 @@ def test_experts_with_weighted_inputs(experts, top, ff, shared, width, n, dtype)
     lw.load(lambda name, shape: W[name].clone(), mcfg, mcfg.layers[0], dtype, torch.device("cuda"))
     h = torch.randn(n, width, generator=torch.Generator().manual_seed(5)).to(dtype)
     a, b = RokevikFeedForward(mcfg.layers[0], lw, False).forward(h.cuda(), None)
-    got = a.float() + (b.float() if b is not None else 0)
+    got = a.float().view(n, -1, width).sum(1) + (b.float() if b is not None else 0)      # (decode-sized: a row per expert)
     want = O.moe_ff(h.double(), f64(W), "l0.mlp.", layer["mlp"])
     e = (got.cpu().double() - want).abs().max(dim=-1).values / want.abs().max()
     if dtype == torch.float32:
@@ -496,7 +503,7 @@ def test_experts_with_weighted_inputs(experts, top, ff, shared, width, n, dtype)
 
 @pytest.mark.parametrize("dtype", [torch.float32, torch.bfloat16, torch.float16])
 def test_gated_unit_with_row_weights(dtype):
-    from swiftllm_amd.worker.kernels.moe import ACT_CLAMPED, gated_unit
+    from swiftllm_amd.worker.kernels.moe import ACT_CLAMPED, ACT_SILU_UP_FIRST, gated_unit
     g = torch.Generator().manual_seed(3)
     for rows, ff in ((7, 40), (5, 33), (300, 8)):
         gu, w = torch.randn(rows, 2 * ff, generator=g).to(dtype), torch.rand(rows, generator=g) + 0.1
@@ -505,10 +512,30 @@ def test_gated_unit_with_row_weights(dtype):
             want = O.silu(z[:, :ff]) * z[:, ff:]
             got = gated_unit(gu.cuda(), ff, in_w=in_w.cuda() if in_w is not None else None)
             assert (got.cpu().double() - want).abs().max() < (1e-5 if dtype == torch.float32 else 4e-2)
+        got = gated_unit(gu.cuda(), ff, ACT_SILU_UP_FIRST)
         z = gu.double()
+        assert (got.cpu().double() - O.silu(z[:, ff:]) * z[:, :ff]).abs().max() < (1e-5 if dtype == torch.float32 else 4e-2)
         a, b = z[:, :ff].clamp(max=1.5), z[:, ff:].clamp(-1.5, 1.5)
         got = gated_unit(gu.cuda(), ff, ACT_CLAMPED, 1.5)
         assert (got.cpu().double() - a * torch.sigmoid(1.702 * a) * (b + 1)).abs().max() < (1e-5 if dtype == torch.float32 else 4e-2)
+
+
+@pytest.mark.parametrize("n,width,ff", [(1, 128, 64), (32, 256, 96), (50, 128, 64), (200, 128, 32), (7, 100, 30)])
+@pytest.mark.parametrize("packed", [True, False])
+def test_fused_silu_unit(n, width, ff, packed):
+    """The one-launch form of the shared expert's first half, the medium and large forms, and the shapes none of them serves."""
+    from swiftllm_amd.worker.kernels.linear import pack_weight, packable
+    from swiftllm_amd.worker.layers.kekapel_layer import _silu_unit
+    g = torch.Generator().manual_seed(n)
+    h = torch.randn(n, width, generator=g).bfloat16()
+    w = (torch.randn(2 * ff, width, generator=g) / width ** 0.5).bfloat16().cuda()
+    if packed and packable(w):
+        pack_weight(w)
+    z = h.double() @ w.cpu().double().T
+    want = z[:, :ff] * O.silu(z[:, ff:])
+    assert (_silu_unit(h.cuda(), w, True).cpu().double() - want).abs().max() < 1e-2 * max(1.0, float(want.abs().max()))
+    got = _silu_unit(h.float().cuda(), w.float(), False)
+    assert (got.cpu().double() - want).abs().max() < 1e-4
 
 
 def test_capped_logits_and_fp32_argmax():

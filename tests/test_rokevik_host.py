@@ -43,6 +43,7 @@ def test_config_refuses_what_cannot_run():
                        ([O.attention_layer(dim=16, rot_dims=7)], {}),
                        ([O.attention_layer(mlp=O.moe(experts=3, top=4))], {}),
                        ([O.attention_layer()], {"groups": 5}),
+                       ([O.attention_layer()], {"streams": 17}),
                        ([O.attention_layer()], {"loop": (0, 2, 2)})):
         with pytest.raises(ValueError):
             RokevikModelConfig(O.make_config(layers=layers, loop=kw.pop("loop", None), **kw))
