@@ -63,6 +63,36 @@ __device__ __forceinline__ float lane_dot2(const T *x, const T *w, int n, int la
     return a;
 }
 
+// The token's row as fp32 in LDS, for the whole workgroup (the caller synchronises).
+template <typename T>
+__device__ __forceinline__ void stage_row(float *dst, const T *src, int n) {
+    if constexpr (sizeof(T) == 2) {
+        if ((n & 7) == 0 && aligned16_dev(src)) {
+            for (int i = threadIdx.x * 8; i < n; i += kMoeThreads * 8) {
+                const vec8_t<T> v = load8(src + i);
+                *reinterpret_cast<float4_t *>(dst + i) = float4_t{to_f(v[0]), to_f(v[1]), to_f(v[2]), to_f(v[3])};
+                *reinterpret_cast<float4_t *>(dst + i + 4) = float4_t{to_f(v[4]), to_f(v[5]), to_f(v[6]), to_f(v[7])};
+            }
+            return;
+        }
+    }
+    for (int i = threadIdx.x; i < n; i += kMoeThreads) dst[i] = to_f(src[i]);
+}
+// Router logit: x . w over n fp32 elements (x in LDS), reduced over the wave; 16 bytes per lane when the rows allow it.
+__device__ __forceinline__ float router_dot(const float *x, const float *w, int n, int lane) {
+    float a = 0.f;
+    if ((n & 3) == 0 && aligned16_dev(w)) {
+#pragma unroll 4
+        for (int i = lane * 4; i < n; i += 64 * 4) {
+            const float4_t u = *reinterpret_cast<const float4_t *>(x + i), v = *reinterpret_cast<const float4_t *>(w + i);
+            a += (u[0] * v[0] + u[1] * v[1]) + (u[2] * v[2] + u[3] * v[3]);
+        }
+    } else {
+        for (int i = lane; i < n; i += 64) a += x[i] * w[i];
+    }
+    return wave_allreduce_sum(a);
+}
+
 // act 0: g' = min(g, limit), u' = clamp(u, +-limit), g' sigmoid(1.702 g') (u' + 1); act 1: silu(g) u; act 2: silu(u) g
 __device__ __forceinline__ float gated_unit(float g, float u, float limit, int act) {
     if (act == 1) return g / (1.0f + expf(-g)) * u;
@@ -76,18 +106,15 @@ template <typename T>
 __global__ __launch_bounds__(kMoeThreads) void moe_route_kernel(int32_t *idx_out, float *w_out, const T *h,
                                                                 const float *router, const float *bias, int width,
                                                                 int experts, int top, int all_scores, float scale) {
-    extern __shared__ float lds[];
+    extern __shared__ __align__(16) float lds[];
     float *hf = lds;                // [width]
     float *logit = lds + width;     // [experts]
     const int64_t t = blockIdx.x;
     const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
-    for (int i = threadIdx.x; i < width; i += kMoeThreads) hf[i] = to_f(h[t * width + i]);
+    stage_row(hf, h + t * width, width);
     __syncthreads();
     for (int e = wave; e < experts; e += kMoeWaves) {
-        const float *wr = router + static_cast<int64_t>(e) * width;
-        float a = 0.f;
-        for (int i = lane; i < width; i += 64) a += hf[i] * wr[i];
-        a = wave_allreduce_sum(a);
+        const float a = router_dot(hf, router + static_cast<int64_t>(e) * width, width, lane);
         if (lane == 0) logit[e] = a + (bias ? bias[e] : 0.f);
     }
     __syncthreads();
@@ -144,7 +171,7 @@ __global__ __launch_bounds__(kMoeThreads) void moe_route_grouped_kernel(int32_t 
                                                                         const float *router, const float *correction,
                                                                         int width, int experts, int top, int count,
                                                                         int keep, int normalize) {
-    extern __shared__ float lds[];
+    extern __shared__ __align__(16) float lds[];
     float *hf = lds;                    // [width]
     float *score = hf + width;          // [experts] s = sigmoid(logit)
     float *choice = score + experts;    // [experts] s + correction; -inf once taken or outside the kept groups
@@ -152,13 +179,10 @@ __global__ __launch_bounds__(kMoeThreads) void moe_route_grouped_kernel(int32_t 
     float *gkeep = gscore + count;      // [count] 1 for the groups whose experts may be chosen
     const int64_t t = blockIdx.x;
     const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
-    for (int i = threadIdx.x; i < width; i += kMoeThreads) hf[i] = to_f(h[t * width + i]);
+    stage_row(hf, h + t * width, width);
     __syncthreads();
     for (int e = wave; e < experts; e += kMoeWaves) {
-        const float *wr = router + static_cast<int64_t>(e) * width;
-        float a = 0.f;
-        for (int i = lane; i < width; i += 64) a += hf[i] * wr[i];
-        a = wave_allreduce_sum(a);
+        const float a = router_dot(hf, router + static_cast<int64_t>(e) * width, width, lane);
         if (lane == 0) {
             const float sc = 1.0f / (1.0f + expf(-a));
             score[e] = sc;
