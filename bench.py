@@ -182,9 +182,9 @@ def _compare_configs(sz, positions, kv_rank=512):
     # windows of 1024, interpolated rotary) / minGRU of the heads' total width, in turn; two streams, norms in two parts; every
     # feed-forward a mixture of Ratilorn's sizes (8 experts of ff / 4, top 2, a shared one), no loop
     kvattn = dict(dim=sz["dim"], vdim=sz["dim"], heads=sz["heads"], kv_heads=sz["kv_heads"], scale=sz["dim"] ** -0.5,
-                  softcap=50.0, rot=dict(base=10000.0, dims=half))
+                  softcap=30.0, rot=dict(base=10000.0, dims=half))
     klat = dict(heads=sz["heads"], dim=sz["dim"], rot_dim=half, vdim=sz["dim"], kv_rank=kv_rank, mask=dict(size=1024),
-                rot=dict(base=500000.0, dims=half, scaling=dict(factor=8.0, original=1024, fast=32.0, slow=1.0)),
+                rot=dict(base=200000.0, dims=half, scaling=dict(factor=4.0, original=2048, fast=24.0, slow=2.0)),
                 scale=(sz["dim"] + half) ** -0.5)
     kmoe = dict(kind="moe", expert=dict(ff=sz["ff"] // 4), router=dict(experts=8, top=2), shared=dict(ff=sz["ff"] // 4))
     kinds = (("attention", kvattn), ("latent_attention", klat), ("latent_attention", klat),

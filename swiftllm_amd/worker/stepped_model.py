@@ -1,6 +1,6 @@
 """SteppedModel — the worker that every design with a token-level step shares.
 
-A design's worker (KekapelModel, LorulixModel) supplies its configuration class, the layout of a block of the pool, its
+A design's worker (KekapelModel, LorulixModel, ...) supplies its configuration class, the layout of a block of the pool, its
 weights and the stack itself (`_run_stack`, `_logits`); everything around the stack lives here and is the same for all of
 them:
 
