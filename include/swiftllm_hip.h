@@ -558,12 +558,16 @@ int swl_window_attn_tiles(void *out, const void *q, const void *k_cache, const v
  *                 are shared out over ceil(H / heads_per_group) workgroups. -1: the rows of a matrix-core tile are sixteen
  *                 HEADS of one token instead of sixteen tokens (requires num_tiles == num_tokens, i.e. every tile is one
  *                 token, num_kv_heads == 1, no talk, no rel): the form for decode steps of heads that share one key head.
+ *   slopes        NULL, or fp32 [num_q_heads]: slopes[h] * (query position - key position) is taken off the (capped) score.
+ *   out_dim       value columns that count (<= vdim, the row size in the pages); out rows are [num_q_heads * out_dim],
+ *   out_stride    elements apart. gate (NULL: none): the result times sigmoid(gate[t * gate_stride + h * out_dim + c]).
  * The tiles form serves more (dim, vdim) pairs without a mixing matrix than with one: ask swl_masked_attn_tiles_supported. */
 int swl_masked_attn(void *out, const void *q, const void *k_cache, const void *v_cache, const int32_t *block_table,
                     const int32_t *tok_seq, const int32_t *tok_pos, const float *talk, const float *rel, int32_t rel_len,
                     int64_t num_tokens, int32_t num_q_heads, int32_t num_kv_heads, int32_t dim, int32_t vdim,
                     int64_t q_tok_stride, int32_t window, float scale, float softcap, int32_t max_blocks_per_seq,
                     int64_t block_stride, int32_t mask_kind, const float *sink, int32_t num_v_heads, int32_t out_f32,
+                    const float *slopes, int32_t out_dim, int64_t out_stride, const void *gate, int64_t gate_stride,
                     int32_t dtype, swl_stream_t stream);
 int swl_masked_attn_tiles_supported(int32_t num_q_heads, int32_t num_kv_heads, int32_t num_v_heads, int32_t dim,
                                     int32_t vdim, int32_t dtype);
@@ -573,8 +577,8 @@ int swl_masked_attn_tiles(void *out, const void *q, const void *k_cache, const v
                           int32_t num_q_heads, int32_t num_kv_heads, int32_t dim, int32_t vdim, int64_t q_tok_stride,
                           int32_t window, float scale, float softcap, int32_t max_blocks_per_seq, int64_t block_stride,
                           int32_t key_splits, float *scratch, int64_t num_tokens, int32_t mask_kind, const float *sink,
-                          int32_t num_v_heads, int32_t out_f32, int32_t heads_per_group, int32_t dtype,
-                          swl_stream_t stream);
+                          int32_t num_v_heads, int32_t out_f32, int32_t heads_per_group, const float *slopes, int32_t out_dim,
+                          int64_t out_stride, const void *gate, int64_t gate_stride, int32_t dtype, swl_stream_t stream);
 
 /* ---- rotary positions on interleaved pairs fused with the paged KV store; gated / combined heads ---------------------------
  * Rotation: dimension 2i of a head is paired with 2i + 1, i < rot_dims / 2; (u, v) at position p becomes
@@ -637,6 +641,9 @@ int swl_moe_expert_stationary(void *out, const void *x, const void *w, const int
                               int32_t dtype, swl_stream_t stream);
 int swl_glu_clamp(void *y, const void *gate_up, const float *in_w, int64_t num_rows, int32_t ff, float limit, int32_t act,
                   int32_t dtype, swl_stream_t stream);
+/* swl_glu_rows: swl_glu_clamp on rows that are column slices: gate elements at gate_up[r * gu_stride], up elements up_off further. */
+int swl_glu_rows(void *y, int64_t y_stride, const void *gate_up, int64_t gu_stride, int64_t up_off, const float *in_w,
+                 int64_t num_rows, int32_t ff, float limit, int32_t act, int32_t dtype, swl_stream_t stream);
 int swl_moe_combine(void *out, const void *rows, const int64_t *where, const float *expert_w, int64_t num_tokens,
                     int32_t width, int32_t top, int32_t dtype, swl_stream_t stream);
 int swl_moe_down_combine(void *out, const void *y, const void *down, const int32_t *expert_idx, const float *expert_w,
@@ -667,7 +674,9 @@ int swl_qknorm_full_store_kv(void *qkv, const float *q_w, const float *k_w, void
  * * w2. m NULL: only the output norm, of rows row_idx when given. Per-sequence state: `state` is the base of the state slots
  * (fp32, slot_stride floats apart); tok_state[t] = slot * 2 + parity, tok_start[t] = position of the first token of t's
  * portion. swl_causal_conv_state: out = (h if add_input) + causal convolution of h over time with w [taps, channels] (fp32),
- * the carried inputs at tail_off inside the slot ([2][taps - 1][channels] floats). dtype may be SWL_F32. */
+ * the carried inputs at tail_off inside the slot ([2][taps - 1][channels] floats). swl_token_shift_mix: out [mixes][T][width],
+ * out[s][t] = h[t] + (h[t - 1] - h[t]) * mu[s], the last input carried like a two-tap convolution's ([2][width] floats).
+ * dtype may be SWL_F32. */
 int swl_gated_add_rmsnorm(float *x, const void *m, const void *m2, const void *m2_gate, int64_t m2_gate_stride,
                           const void *r, int64_t r_stride, const float *r_bias, const float *w1, void *out, const float *w2,
                           const int32_t *row_idx, float eps, int64_t num_rows, int32_t width, int32_t dtype,
@@ -676,6 +685,10 @@ int swl_causal_conv_state(void *out, int64_t out_stride, const void *h, int64_t 
                           int64_t slot_stride, int64_t tail_off, const int32_t *tok_pos, const int32_t *tok_start,
                           const int32_t *tok_state, const int32_t *tok_seq, int64_t num_tokens, int32_t channels,
                           int32_t taps, int32_t add_input, int32_t dtype, swl_stream_t stream);
+int swl_token_shift_mix(void *out, const void *h, int64_t h_stride, const float *mu, int32_t mixes, float *state,
+                        int64_t slot_stride, int64_t tail_off, const int32_t *tok_pos, const int32_t *tok_start,
+                        const int32_t *tok_state, const int32_t *tok_seq, int64_t num_tokens, int32_t width, int32_t dtype,
+                        swl_stream_t stream);
 
 /* ---- gated delta rule (csrc/delta_rule.hip) --------------------------------------------------------------------------------
  * swl_delta_prep: proj rows [q | k | v | gate | b | a] -> qn, kn [T, qk heads * dim], kq [T, qk heads] (their dot
@@ -683,7 +696,8 @@ int swl_causal_conv_state(void *out, int64_t out_stride, const void *h, int64_t 
  * [T, heads], all fp32 (convolution + SiLU with conv_w tap-major [taps, q | k | v channels], unit norms, sigmoid,
  * exp(-exp(A_log) softplus(a + dt_bias))).
  * swl_delta_rule: o[T, heads * vdim] (fp32) and the states [heads, dim, vdim] at s_off inside the slots, one portion per
- * (seq_row0, seq_cnt) entry. swl_gated_head_rmsnorm: out = o / rms(o over vdim) * w[vdim] * silu(gate). */
+ * (seq_row0, seq_cnt) entry. swl_gated_head_rmsnorm: out[t * out_stride + h * vdim + e] = mult * o / rms(o over vdim) *
+ * w[h * w_head_stride + e] * silu(gate) (w_head_stride 0: one weight row for all heads). */
 int swl_delta_prep(float *qn, float *kn, float *kq, float *vv, float *beta, float *decay, const void *proj, int64_t proj_stride,
                    const float *conv_w, const float *a_log, const float *dt_bias, float *state, int64_t slot_stride,
                    int64_t tail_off, const int32_t *tok_pos, const int32_t *tok_start, const int32_t *tok_state,
@@ -693,8 +707,8 @@ int swl_delta_rule(float *o, const float *qn, const float *kn, const float *kq, 
                    float *state, int64_t slot_stride, int64_t s_off, const int32_t *seq_row0, const int32_t *seq_cnt,
                    const int32_t *tok_pos, const int32_t *tok_state, int32_t num_seqs, int32_t num_heads,
                    int32_t num_qk_heads, int32_t dim, int32_t vdim, swl_stream_t stream);
-int swl_gated_head_rmsnorm(void *out, const float *o, const void *gate, int64_t gate_stride, const float *w, float eps,
-                           int64_t num_tokens, int32_t num_heads, int32_t vdim, int32_t dtype, swl_stream_t stream);
+int swl_gated_head_rmsnorm(void *out, int64_t out_stride, const float *o, const void *gate, int64_t gate_stride, const float *w,
+                           int32_t w_head_stride, float mult, float eps, int64_t num_tokens, int32_t num_heads, int32_t vdim, int32_t dtype, swl_stream_t stream);
 
 /* ---- sigmoid router with group-limited choice (csrc/moe.hip) ---------------------------------------------------------------
  * s = sigmoid(router[experts, width] h) in fp32. Experts are chosen by s + correction (NULL: by s): the experts form
@@ -752,7 +766,7 @@ int swl_ssd_scan(float *y, const float *xbc, const float *dt, const float *decay
                  int64_t slot_stride, int64_t s_off, const int32_t *seq_row0, const int32_t *seq_cnt, const int32_t *tok_pos,
                  const int32_t *tok_state, int32_t num_seqs, int32_t num_heads, int32_t vdim, int32_t state_dim,
                  int32_t groups, swl_stream_t stream);
-int swl_gated_group_rmsnorm(void *out, const float *y, const void *gate, int64_t gate_stride, const float *w, float eps,
+int swl_gated_group_rmsnorm(void *out, int64_t out_stride, const float *y, const void *gate, int64_t gate_stride, const float *w, float eps,
                             int64_t num_tokens, int32_t cols, int32_t groups, int32_t dtype, swl_stream_t stream);
 
 /* ---- fp32 stream of models that norm a sublayer's RESULT only (csrc/rms_stream.hip) -----------------------------------------
@@ -776,6 +790,50 @@ int swl_qk_norm_rope_store_kv(const void *rows, void *q_out, const float *q_b, c
                               int32_t rot_dims, int32_t half, double rot_mult, int64_t tok_stride, int64_t q_out_stride,
                               int32_t k_dim, int32_t v_dim, int32_t keys_as_values, int32_t max_blocks_per_seq,
                               int64_t block_stride, float eps, int32_t dtype, swl_stream_t stream);
+
+/* rows [q | k | v] -> bias [q | k | v] (fp32, NULL: none), causal convolution (conv_w tap-major [taps, q | k | v channels] fp32,
+ * NULL: none; zeros before the sequence; carried inputs [2][taps - 1][channels] at tail_off inside the slot), RMS norm of the q / k
+ * heads with q_w / k_w [dim] (NULL: none), rotation (rot_dims 0: none); q to q_out (heads k_dim apart), k to the K pool, v_mult * v
+ * to the V pool, rows of k_dim / v_dim with zeros beyond the head. k_cache NULL: queries only. dtype may be SWL_F32. */
+int swl_qkv_conv_rope_store_kv(
+    const void *rows, int64_t tok_stride, void *q_out, int64_t q_out_stride, const float *bias, const float *conv_w, int32_t taps,
+    const float *q_w, const float *k_w, const double *freq, int32_t rot_dims, int32_t half, double rot_mult, float v_mult,
+    void *k_cache, void *v_cache, const int32_t *block_table, int32_t max_blocks_per_seq, int64_t block_stride, float *state,
+    int64_t slot_stride, int64_t tail_off, const int32_t *tok_pos, const int32_t *tok_start, const int32_t *tok_state,
+    const int32_t *tok_seq, int64_t num_tokens, int32_t num_q_heads, int32_t num_kv_heads, int32_t dim, int32_t vdim, int32_t k_dim,
+    int32_t v_dim, float eps, int32_t dtype, swl_stream_t stream);
+
+/* ---- recurrences linear in a matrix state (csrc/linear_scan.hip) -----------------------------------------------------------------
+ * Per head: S <- diag(a) S + k v^T, o = S^T q (+ dskip v); with bonus [heads, dim]: o = (S + diag(bonus) k v^T)^T q before the
+ * update. q (times q_scale) and k (times k_scale[t][h], NULL: 1) have num_qk_heads heads of dim, shared by num_heads / num_qk_heads
+ * heads each; decay fp32, one per channel ([t][heads * dim]) or per head ([t][heads]). States [heads, dim, vdim] fp32 at s_off
+ * inside the slots.
+ * swl_linear_chunks prepares tiles of up to 16 tokens, dp = dim rounded up to 16: qd [tiles, heads, 16, dp], kd [tiles, heads, dp,
+ * 16], total [tiles, heads, dp], intra [tiles, heads, 16, 16]; swl_linear_scan walks every portion's tiles (the first is
+ * seq_tile0[s]) and writes o fp32. dim <= 320. swl_linear_step: portions of one token: y fp32 (NULL: not wanted) and / or out =
+ * mult * o / rms(o over vdim) * norm_w[h * norm_head_stride + c] * silu(gate) in dtype. dtype (of q, k, v, gate, out) may be SWL_F32. */
+int swl_linear_chunks(float *qd, float *kd, float *total, float *intra, const void *q, int64_t q_stride, const void *k,
+                      int64_t k_stride, const float *decay, int64_t decay_stride, int32_t per_channel, const float *k_scale,
+                      const float *bonus, float q_scale, const int32_t *tile_row0, const int32_t *tile_cnt, int32_t num_tiles,
+                      int32_t num_heads, int32_t num_qk_heads, int32_t dim, int32_t dtype, swl_stream_t stream);
+int swl_linear_scan(float *o, int64_t o_stride, const float *qd, const float *kd, const float *total, const float *intra,
+                    const void *v, int64_t v_stride, const float *dskip, float *state, int64_t slot_stride, int64_t s_off,
+                    const int32_t *seq_row0, const int32_t *seq_cnt, const int32_t *seq_tile0, const int32_t *tok_pos,
+                    const int32_t *tok_state, int32_t num_seqs, int32_t num_heads, int32_t dim, int32_t vdim, int32_t dtype,
+                    swl_stream_t stream);
+int swl_linear_step(void *out, int64_t out_stride, float *y, int64_t y_stride, const void *q, int64_t q_stride, const void *k,
+                    int64_t k_stride, const void *v, int64_t v_stride, const float *decay, int64_t decay_stride,
+                    int32_t per_channel, const float *k_scale, const float *bonus, float q_scale, const float *dskip, float *state,
+                    int64_t slot_stride, int64_t s_off, const int32_t *seq_row0, const int32_t *tok_pos, const int32_t *tok_state,
+                    int32_t num_seqs, int32_t num_heads, int32_t num_qk_heads, int32_t dim, int32_t vdim, const float *norm_w,
+                    int32_t norm_head_stride, const void *gate, int64_t gate_stride, float eps, float mult, int32_t dtype,
+                    swl_stream_t stream);
+
+/* out fp32 [T, channels] = sigmoid(y)^power (kind 0) or exp(-exp(y)) (kind 1), y = w2 z + bias, z = act(w1 x) (act 0: identity,
+ * 1: tanh; w1 NULL: z = act(x)); w1 [rank, width], w2 [channels, rank]; rank <= 256 (csrc/low_rank_decay.hip). dtype may be SWL_F32. */
+int swl_low_rank_decay(float *out, const void *x, int64_t x_stride, const void *w1, const void *w2, const float *bias,
+                       int64_t num_tokens, int32_t width, int32_t rank, int32_t channels, int32_t act, int32_t kind, float power,
+                       int32_t dtype, swl_stream_t stream);
 
 /* ---- fp32 residual of several streams, hyper-connections (csrc/hyper_stream.hip) ------------------------------------------------
  * x [rows, streams, width] fp32. swl_embed_streams: every stream = embed[token]. swl_hyper_step: with y (+ y2, + y_bias[width])

@@ -104,9 +104,10 @@ SIGNATURES = {
     "swl_window_attn_tiles": [_P, _P, _P, _P, _P, _P, _P, _P, _P, _P, _P, _I32, _I32, _I32, _I32, _I32, _I32, _I64, _I32, _F32, _F32,
                               _I32, _I64, _I32, _P, _I64, _I32, _P],
     "swl_masked_attn": [_P, _P, _P, _P, _P, _P, _P, _P, _P, _I32, _I64, _I32, _I32, _I32, _I32, _I64, _I32, _F32, _F32, _I32,
-                        _I64, _I32, _P, _I32, _I32, _I32, _P],
-    "swl_masked_attn_tiles": [_P, _P, _P, _P, _P, _P, _P, _P, _P, _P, _P, _I32, _I32, _I32, _I32, _I32, _I32, _I64, _I32, _F32,
-                              _F32, _I32, _I64, _I32, _P, _I64, _I32, _P, _I32, _I32, _I32, _I32, _P],
+                        _I64, _I32, _P, _I32, _I32, _P, _I32, _I64, _P, _I64, _I32, _P],
+    "swl_masked_attn_tiles": [_P, _P, _P, _P, _P, _P, _P, _P, _P, _P, _P, _I32, _I32, _I32, _I32, _I32, _I32, _I64, _I32,
+                              _F32, _F32, _I32, _I64, _I32, _P, _I64, _I32, _P, _I32, _I32, _I32, _P, _I32, _I64, _P, _I64,
+                              _I32, _P],
     "swl_rope_store_kv": [_P, _P, _P, _P, _P, _P, _P, _I64, _I32, _I32, _I32, _I32, _I32, _I32, _I64, _I32, _I64, _I32, _P],
     "swl_latent_rope_store_kv": [_P, _P, _P, _P, _P, _P, _P, _P, _P, _I64, _I32, _I32, _I32, _I32, _I64, _I64, _I64, _I32,
                                  _I64, _F32, _I32, _F64, _I32, _I32, _I32, _P],
@@ -129,7 +130,7 @@ SIGNATURES = {
     "swl_delta_prep": [_P, _P, _P, _P, _P, _P, _P, _I64, _P, _P, _P, _P, _I64, _I64, _P, _P, _P, _P, _I64, _I32, _I32, _I32,
                        _I32, _I32, _I32, _P],
     "swl_delta_rule": [_P, _P, _P, _P, _P, _P, _P, _P, _I64, _I64, _P, _P, _P, _P, _I32, _I32, _I32, _I32, _I32, _P],
-    "swl_gated_head_rmsnorm": [_P, _P, _P, _I64, _P, _F32, _I64, _I32, _I32, _I32, _P],
+    "swl_gated_head_rmsnorm": [_P, _I64, _P, _P, _I64, _P, _I32, _F32, _F32, _I64, _I32, _I32, _I32, _P],
     "swl_moe_route_grouped": [_P, _P, _P, _P, _P, _I64, _I32, _I32, _I32, _I32, _I32, _I32, _I32, _P],
     "swl_qkv_bias_norm_store": [_P, _P, _P, _P, _P, _P, _P, _I64, _F32, _P, _P, _P, _P, _P, _I64, _I32, _I32, _I32, _I32,
                                 _I64, _I32, _I64, _F32, _I32, _P],
@@ -140,7 +141,7 @@ SIGNATURES = {
     "swl_ssd_prep": [_P, _P, _P, _P, _I64, _P, _P, _P, _P, _P, _I64, _I64, _P, _P, _P, _P, _I64, _I32, _I32, _I32, _I32,
                      _I32, _I32, _P],
     "swl_ssd_scan": [_P, _P, _P, _P, _P, _P, _I64, _I64, _P, _P, _P, _P, _I32, _I32, _I32, _I32, _I32, _P],
-    "swl_gated_group_rmsnorm": [_P, _P, _P, _I64, _P, _F32, _I64, _I32, _I32, _I32, _P],
+    "swl_gated_group_rmsnorm": [_P, _I64, _P, _P, _I64, _P, _F32, _I64, _I32, _I32, _I32, _P],
     "swl_logit_softcap": [_P, _P, _I64, _F32, _I32, _P],
     "swl_qk_norm_rope_store_kv": [_P, _P, _P, _P, _P, _P, _P, _P, _P, _P, _P, _P, _P, _I64, _I32, _I32, _I32, _I32, _I32, _I32,
                                   _I32, _F64, _I64, _I64, _I32, _I32, _I32, _I32, _I64, _F32, _I32, _P],
@@ -150,6 +151,18 @@ SIGNATURES = {
     "swl_min_gru_carry": [_P, _P, _I64, _I64, _P, _P, _P, _P, _P, _I32, _I32, _I32, _P],
     "swl_min_gru_apply": [_P, _P, _I64, _P, _P, _P, _P, _I64, _I64, _P, _P, _P, _P, _I32, _I32, _I32, _P],
     "swl_post_norm_add": [_P, _P, _P, _P, _P, _F32, _P, _P, _P, _F32, _I64, _I32, _I32, _P],
+    "swl_glu_rows": [_P, _I64, _P, _I64, _I64, _P, _I64, _I32, _F32, _I32, _I32, _P],
+    "swl_token_shift_mix": [_P, _P, _I64, _P, _I32, _P, _I64, _I64, _P, _P, _P, _P, _I64, _I32, _I32, _P],
+    "swl_qkv_conv_rope_store_kv": [_P, _I64, _P, _I64, _P, _P, _I32, _P, _P, _P, _I32, _I32, _F64, _F32, _P, _P, _P, _I32,
+                                   _I64, _P, _I64, _I64, _P, _P, _P, _P, _I64, _I32, _I32, _I32, _I32, _I32, _I32, _F32,
+                                   _I32, _P],
+    "swl_linear_chunks": [_P, _P, _P, _P, _P, _I64, _P, _I64, _P, _I64, _I32, _P, _P, _F32, _P, _P, _I32, _I32, _I32, _I32,
+                          _I32, _P],
+    "swl_linear_scan": [_P, _I64, _P, _P, _P, _P, _P, _I64, _P, _P, _I64, _I64, _P, _P, _P, _P, _P, _I32, _I32, _I32, _I32,
+                        _I32, _P],
+    "swl_linear_step": [_P, _I64, _P, _I64, _P, _I64, _P, _I64, _P, _I64, _P, _I64, _I32, _P, _P, _F32, _P, _P, _I64, _I64,
+                        _P, _P, _P, _I32, _I32, _I32, _I32, _I32, _P, _I32, _P, _I64, _F32, _F32, _I32, _P],
+    "swl_low_rank_decay": [_P, _P, _I64, _P, _P, _P, _I64, _I32, _I32, _I32, _I32, _I32, _F32, _I32, _P],
 }
 # Entry points that do not follow the "int rc = f(...)" convention.
 _SPECIAL = {

@@ -42,6 +42,8 @@ SOURCES = [
     "ssd.hip",
     "hyper_stream.hip",
     "min_gru.hip",
+    "linear_scan.hip",
+    "low_rank_decay.hip",
 ]
 # What a model family's worker calls (the shared pieces included): `build(only=MODEL_SOURCES[...])` compiles just these, so
 # that the first use from a fresh checkout does not pay for kernels the model never launches. A later full build compiles
@@ -58,6 +60,8 @@ MODEL_SOURCES = {
     "Ratilorn": _SHARED + ["layernorm.hip", "qknorm_kv.hip", "window_attn.hip", "window_attn_mfma.hip", "moe.hip",
                            "rms_stream.hip", "sigmoid_attn.hip", "ssd.hip"],
     "Rokevik": _SHARED + ["window_attn.hip", "window_attn_mfma.hip", "moe.hip", "rope_kv.hip", "hyper_stream.hip", "min_gru.hip"],
+    "Vafozen": _SHARED + ["layernorm.hip", "window_attn.hip", "window_attn_mfma.hip", "moe.hip", "rms_stream.hip", "rope_kv.hip",
+                          "hyper_stream.hip", "delta_rule.hip", "ssd.hip", "linear_scan.hip", "low_rank_decay.hip"],
 }
 HEADERS = ["swl_common.h", "attend_block.h", "conv_tail.h", os.path.join(ROOT, "include", "swiftllm_hip.h")]
 LIB = os.path.join(HERE, "libswiftllm_hip.so")

@@ -14,7 +14,7 @@
 //                    sequential whatever the cut of the sequence into steps: the same operations in the same order. When
 //                    a step has few (portion, head) pairs the columns of a head are shared out over several workgroups. A
 //                    wave of loaders stages the next 16 tokens into a second LDS buffer while the others walk the current ones.
-//   swl_gated_head_rmsnorm: out = o / rms(o over vdim) * w * silu(gate), per head.
+//   swl_gated_head_rmsnorm: out = c * o / rms(o over vdim) * w * silu(gate), per head; w is shared by the heads or one row per head.
 #include "swl_common.h"
 #include "conv_tail.h"
 
@@ -245,7 +245,8 @@ __global__ __launch_bounds__(1024) void delta_rule_kernel(float *o, const float 
 
 template <typename T>
 __global__ __launch_bounds__(256) void gated_head_rmsnorm_kernel(T *out, const float *o, const T *gate, int64_t gate_stride,
-                                                                 const float *w, float eps, int H, int dv) {
+                                                                 const float *w, int w_head_stride, float mult, float eps, int H,
+                                                                 int dv, int64_t out_stride) {
     const int64_t t = blockIdx.x;
     const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
     for (int h = wave; h < H; h += 4) {
@@ -253,10 +254,10 @@ __global__ __launch_bounds__(256) void gated_head_rmsnorm_kernel(T *out, const f
         float ss = 0.f;
         for (int e = lane; e < dv; e += 64) ss += src[e] * src[e];
         ss = wave_allreduce_sum(ss);
-        const float r = 1.0f / sqrtf(ss / static_cast<float>(dv) + eps);
+        const float r = mult / sqrtf(ss / static_cast<float>(dv) + eps);
         for (int e = lane; e < dv; e += 64) {
             const float z = to_f(gate[t * gate_stride + h * dv + e]);
-            out[(t * H + h) * dv + e] = to_t<T>(src[e] * r * w[e] * (z * dr_sigmoid(z)));
+            out[t * out_stride + h * dv + e] = to_t<T>(src[e] * r * w[static_cast<int64_t>(h) * w_head_stride + e] * (z * dr_sigmoid(z)));
         }
     }
 }
@@ -359,10 +360,11 @@ extern "C" int swl_delta_rule(float *o, const float *qn, const float *kn, const 
     return SWL_ERR_UNSUPPORTED;
 }
 
-extern "C" int swl_gated_head_rmsnorm(void *out, const float *o, const void *gate, int64_t gate_stride, const float *w,
-                                      float eps, int64_t num_tokens, int32_t num_heads, int32_t vdim, int32_t dtype,
+extern "C" int swl_gated_head_rmsnorm(void *out, int64_t out_stride, const float *o, const void *gate, int64_t gate_stride,
+                                      const float *w, int32_t w_head_stride, float mult, float eps, int64_t num_tokens, int32_t num_heads, int32_t vdim, int32_t dtype,
                                       swl_stream_t stream) {
-    if (num_tokens < 0 || num_heads <= 0 || vdim <= 0 || gate_stride < static_cast<int64_t>(num_heads) * vdim)
+    if (num_tokens < 0 || num_heads <= 0 || vdim <= 0 || gate_stride < static_cast<int64_t>(num_heads) * vdim ||
+        out_stride < static_cast<int64_t>(num_heads) * vdim)
         return SWL_ERR_BAD_ARG;
     if (num_tokens == 0) return SWL_OK;
     if (!out || !o || !gate || !w) return SWL_ERR_BAD_ARG;
@@ -370,7 +372,7 @@ extern "C" int swl_gated_head_rmsnorm(void *out, const float *o, const void *gat
     SWL_DISPATCH_DTYPE3(dtype, T, {
         hipLaunchKernelGGL((swl::gated_head_rmsnorm_kernel<T>), dim3(static_cast<unsigned>(num_tokens)), dim3(256), 0,
                            static_cast<hipStream_t>(stream), static_cast<T *>(out), o, static_cast<const T *>(gate),
-                           gate_stride, w, eps, num_heads, vdim);
+                           gate_stride, w, w_head_stride, mult, eps, num_heads, vdim, out_stride);
     });
     return swl::check_launch();
 }

@@ -525,30 +525,32 @@ __global__ __launch_bounds__(kMoeThreads, 2) void moe_expert_stationary_kernel(T
 // y[r][f] = act(w[r] gu[r][f], w[r] gu[r][ff + f]) for rows of [gate | up] products that came from a library GEMM (in_w NULL: 1)
 template <typename T>
 __global__ __launch_bounds__(kMoeThreads) void glu_clamp_kernel(T *y, const T *gu, const float *in_w, int64_t total, int ff,
-                                                                float limit, int act) {
+                                                                float limit, int act, int64_t y_stride, int64_t gu_stride,
+                                                                int64_t up_off) {
     const int64_t i = static_cast<int64_t>(blockIdx.x) * kMoeThreads + threadIdx.x;
     if (i >= total) return;
     const int64_t r = i / ff;
     const int f = static_cast<int>(i - r * ff);
     const float w = in_w ? in_w[r] : 1.f;
-    y[i] = to_t<T>(gated_unit(w * to_f(gu[r * 2 * ff + f]), w * to_f(gu[r * 2 * ff + ff + f]), limit, act));
+    const T *g = gu + r * gu_stride + f;
+    y[r * y_stride + f] = to_t<T>(gated_unit(w * to_f(g[0]), w * to_f(g[up_off]), limit, act));
 }
 
 // the same for 16-bit rows of a multiple of 8 elements on 16-byte boundaries: 8 elements (16 bytes) per lane
 template <typename T>
 __global__ __launch_bounds__(kMoeThreads) void glu_clamp_wide_kernel(T *y, const T *gu, const float *in_w, int64_t total8,
-                                                                     int ff8, float limit, int act) {
+                                                                     int ff8, float limit, int act, int64_t y_stride,
+                                                                     int64_t gu_stride, int64_t up_off) {
     const int64_t i = static_cast<int64_t>(blockIdx.x) * kMoeThreads + threadIdx.x;
     if (i >= total8) return;
     const int64_t r = i / ff8;
     const int f = static_cast<int>(i - r * ff8) * 8;
-    const int64_t ff = static_cast<int64_t>(ff8) * 8;
     const float w = in_w ? in_w[r] : 1.f;
-    const vec8_t<T> g = load8(gu + r * 2 * ff + f), u = load8(gu + r * 2 * ff + ff + f);
+    const vec8_t<T> g = load8(gu + r * gu_stride + f), u = load8(gu + r * gu_stride + up_off + f);
     vec8_t<T> o;
 #pragma unroll
     for (int j = 0; j < 8; ++j) o[j] = to_t<T>(gated_unit(w * to_f(g[j]), w * to_f(u[j]), limit, act));
-    store8(y + r * ff + f, o);
+    store8(y + r * y_stride + f, o);
 }
 
 // out[t] = sum_j w[t][j] * rows[where[t * top + j]]  (fp32 sum in the order j = 0, 1, ...)
@@ -613,12 +615,14 @@ extern "C" int swl_moe_expert_stationary(void *out, const void *x, const void *w
     return swl::check_launch();
 }
 
-extern "C" int swl_glu_clamp(void *y, const void *gate_up, const float *in_w, int64_t num_rows, int32_t ff, float limit,
-                             int32_t act, int32_t dtype, swl_stream_t stream) {
-    if (num_rows < 0 || ff <= 0 || act < 0 || act > 2) return SWL_ERR_BAD_ARG;
+extern "C" int swl_glu_rows(void *y, int64_t y_stride, const void *gate_up, int64_t gu_stride, int64_t up_off, const float *in_w,
+                            int64_t num_rows, int32_t ff, float limit, int32_t act, int32_t dtype, swl_stream_t stream) {
+    if (num_rows < 0 || ff <= 0 || act < 0 || act > 2 || y_stride < ff || up_off < ff || gu_stride < up_off + ff)
+        return SWL_ERR_BAD_ARG;
     if (num_rows == 0) return SWL_OK;
     if (!y || !gate_up) return SWL_ERR_BAD_ARG;
-    const bool wide = dtype != SWL_F32 && ff % 8 == 0 && swl::aligned16(y) && swl::aligned16(gate_up);
+    const bool wide = dtype != SWL_F32 && ((ff | y_stride | gu_stride | up_off) & 7) == 0 && swl::aligned16(y) &&
+                      swl::aligned16(gate_up);
     const int64_t total = num_rows * ff / (wide ? 8 : 1);
     const int64_t blocks = (total + swl::kMoeThreads - 1) / swl::kMoeThreads;
     if (blocks > 0x7fffffffLL) return SWL_ERR_UNSUPPORTED;
@@ -626,16 +630,21 @@ extern "C" int swl_glu_clamp(void *y, const void *gate_up, const float *in_w, in
         SWL_DISPATCH_DTYPE(dtype, T, {
             hipLaunchKernelGGL((swl::glu_clamp_wide_kernel<T>), dim3(static_cast<unsigned>(blocks)), dim3(swl::kMoeThreads), 0,
                                static_cast<hipStream_t>(stream), static_cast<T *>(y), static_cast<const T *>(gate_up), in_w,
-                               total, ff / 8, limit, act);
+                               total, ff / 8, limit, act, y_stride, gu_stride, up_off);
         });
         return swl::check_launch();
     }
     SWL_DISPATCH_DTYPE3(dtype, T, {
         hipLaunchKernelGGL((swl::glu_clamp_kernel<T>), dim3(static_cast<unsigned>(blocks)), dim3(swl::kMoeThreads), 0,
                            static_cast<hipStream_t>(stream), static_cast<T *>(y), static_cast<const T *>(gate_up), in_w, total,
-                           ff, limit, act);
+                           ff, limit, act, y_stride, gu_stride, up_off);
     });
     return swl::check_launch();
+}
+
+extern "C" int swl_glu_clamp(void *y, const void *gate_up, const float *in_w, int64_t num_rows, int32_t ff, float limit,
+                             int32_t act, int32_t dtype, swl_stream_t stream) {
+    return swl_glu_rows(y, ff, gate_up, 2 * static_cast<int64_t>(ff), ff, in_w, num_rows, ff, limit, act, dtype, stream);
 }
 
 extern "C" int swl_moe_combine(void *out, const void *rows, const int64_t *where, const float *expert_w,

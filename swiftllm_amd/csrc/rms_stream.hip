@@ -18,6 +18,8 @@
 //     one sequence, for any cut of the sequence into steps: inputs of earlier steps come from the sequence's state slot,
 //     which keeps the last taps - 1 inputs. The tail is double-buffered: a step reads buffer `parity` and the workgroup of
 //     a portion's last token writes the other one, so no launch reads what it writes.
+//   swl_token_shift_mix: out[s][t] = h[t] + (h[t - 1] - h[t]) * mu[s] for several mixing vectors at once (h[-1] = 0); the last input
+//     of every sequence is carried like a two-tap convolution's.
 #include "swl_common.h"
 #include "conv_tail.h"
 
@@ -155,6 +157,43 @@ __global__ __launch_bounds__(kRsThreads) void causal_conv_state_kernel(
     }
 }
 
+template <typename T>
+__global__ __launch_bounds__(kRsThreads) void token_shift_mix_kernel(
+    T *out, int64_t plane, const T *h, int64_t h_stride, const float *mu, int mixes, float *state, int64_t slot_stride,
+    int64_t tail_off, const int32_t *tok_pos, const int32_t *tok_start, const int32_t *tok_state, const int32_t *tok_seq,
+    int64_t num_tokens, int C) {
+    const int64_t t = blockIdx.x;
+    const ConvTail tail(state, slot_stride, tail_off, tok_pos, tok_start, tok_state, tok_seq, num_tokens, C, 2, t);
+    if constexpr (sizeof(T) == 2) {
+        if (ConvTail::wide_ok(h, h_stride, mu, state, slot_stride, tail_off, C) && (plane & 7) == 0 &&
+            (reinterpret_cast<uintptr_t>(out) & 15) == 0) {
+            for (int c = threadIdx.x * 8; c < C; c += kRsThreads * 8) {
+                const vec8_t<T> x = load8(h + t * h_stride + c);
+                float cur[8], prev[8];
+#pragma unroll
+                for (int j = 0; j < 8; ++j) cur[j] = to_f(x[j]);
+                tail.at8(h, h_stride, c, tail.pos - 1, prev);
+                for (int s = 0; s < mixes; ++s) {
+                    const float4_t m0 = *reinterpret_cast<const float4_t *>(mu + static_cast<int64_t>(s) * C + c);
+                    const float4_t m1 = *reinterpret_cast<const float4_t *>(mu + static_cast<int64_t>(s) * C + c + 4);
+                    vec8_t<T> o;
+#pragma unroll
+                    for (int j = 0; j < 8; ++j) o[j] = to_t<T>(cur[j] + (prev[j] - cur[j]) * (j < 4 ? m0[j & 3] : m1[j & 3]));
+                    store8(out + s * plane + t * C + c, o);
+                }
+                tail.save8(h, h_stride, c, cur);
+            }
+            return;
+        }
+    }
+    for (int c = threadIdx.x; c < C; c += kRsThreads) {
+        const float cur = to_f(h[t * h_stride + c]), prev = tail.at(h, h_stride, c, tail.pos - 1);
+        for (int s = 0; s < mixes; ++s)
+            out[s * plane + t * C + c] = to_t<T>(cur + (prev - cur) * mu[static_cast<int64_t>(s) * C + c]);
+        tail.save(h, h_stride, c, cur);
+    }
+}
+
 inline size_t rs_lds_bytes(int width) { return (static_cast<size_t>(width) + kRsThreads / 64) * sizeof(float); }
 
 } // namespace swl
@@ -193,6 +232,23 @@ extern "C" int swl_causal_conv_state(void *out, int64_t out_stride, const void *
                            dim3(swl::kRsThreads), 0, static_cast<hipStream_t>(stream), static_cast<T *>(out), out_stride,
                            static_cast<const T *>(h), h_stride, w, state, slot_stride, tail_off, tok_pos, tok_start,
                            tok_state, tok_seq, num_tokens, channels, taps, add_input);
+    });
+    return swl::check_launch();
+}
+
+extern "C" int swl_token_shift_mix(void *out, const void *h, int64_t h_stride, const float *mu, int32_t mixes, float *state,
+                                   int64_t slot_stride, int64_t tail_off, const int32_t *tok_pos, const int32_t *tok_start,
+                                   const int32_t *tok_state, const int32_t *tok_seq, int64_t num_tokens, int32_t width,
+                                   int32_t dtype, swl_stream_t stream) {
+    if (num_tokens < 0 || width <= 0 || mixes <= 0 || h_stride < width) return SWL_ERR_BAD_ARG;
+    if (num_tokens == 0) return SWL_OK;
+    if (!out || !h || !mu || !state || !tok_pos || !tok_start || !tok_state || !tok_seq) return SWL_ERR_BAD_ARG;
+    if (num_tokens > 0x7fffffffLL) return SWL_ERR_UNSUPPORTED;
+    SWL_DISPATCH_DTYPE3(dtype, T, {
+        hipLaunchKernelGGL((swl::token_shift_mix_kernel<T>), dim3(static_cast<unsigned>(num_tokens)), dim3(swl::kRsThreads), 0,
+                           static_cast<hipStream_t>(stream), static_cast<T *>(out), num_tokens * width,
+                           static_cast<const T *>(h), h_stride, mu, mixes, state, slot_stride, tail_off, tok_pos, tok_start,
+                           tok_state, tok_seq, num_tokens, width);
     });
     return swl::check_launch();
 }

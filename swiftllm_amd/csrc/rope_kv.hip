@@ -13,6 +13,10 @@
 //   swl_qk_norm_rope_store_kv rows [q | k (| v)] of a projection whose biases are still to be added: per head bias, weighted RMS norm,
 //                             rotation; q times a factor per head into a buffer of its own, k into the K pool, and into the V
 //                             pool either the value columns or the KEYS AS PROJECTED (bias added, neither normed nor rotated).
+//   swl_qkv_conv_rope_store_kv  rows [q | k | v] of a projection whose biases are still to be added, each step optional: bias, causal
+//                             convolution over time per channel (inputs of earlier steps carried as projected, conv_tail.h),
+//                             weighted RMS norm of the q / k heads, rotation; q into a buffer of its own, k into the K pool, v
+//                             times a constant into the V pool. The row passes through LDS in fp32 and is rounded once.
 //   swl_latent_rope_store_kv  latent attention. Rows hold H query heads [d unrotated | dr rotated] and (optionally) the
 //                             compressed key/value row [r latent | dr shared rotated key part]. The rotated query parts go
 //                             to qa[t][h][r : r + dr] (the caller fills qa[t][h][0 : r] with the queries folded through
@@ -28,6 +32,7 @@
 // middle may lay heads out wider than they are (k_dim, v_dim: the row sizes that a compiled attention kernel serves); the
 // columns beyond the head are written as zeros, which neither scores nor outputs see.
 #include "swl_common.h"
+#include "conv_tail.h"
 
 namespace swl {
 
@@ -261,6 +266,130 @@ __global__ __launch_bounds__(kRkThreads) void qk_norm_rope_store_kv_kernel(
 }
 
 template <typename T>
+__global__ __launch_bounds__(kRkThreads) void qkv_conv_rope_store_kv_kernel(
+    const T *rows, int64_t tok_stride, T *q_out, int64_t q_out_stride, const float *bias, const float *conv_w, int taps,
+    const float *q_w, const float *k_w, const double *freq, int rot_dims, int half, double rot_mult, float v_mult, T *k_cache,
+    T *v_cache, const int32_t *block_table, int max_blocks_per_seq, int64_t block_stride, float *state, int64_t slot_stride,
+    int64_t tail_off, const int32_t *tok_pos, const int32_t *tok_start, const int32_t *tok_state, const int32_t *tok_seq,
+    int64_t num_tokens, int nq, int nk, int d, int dv, int k_dim, int v_dim, float eps) {
+    extern __shared__ float act[];      // [(nq + nk) d + nk dv] biased, convolved channels; then [nq + nk] the heads' 1 / rms
+    __shared__ float cs[kRkMaxPairs], sn[kRkMaxPairs];
+    const int64_t t = blockIdx.x;
+    const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
+    const int pos = tok_pos[t];
+    const int pairs = rot_dims >> 1, heads = nq + nk, C = heads * d + nk * dv;
+    float *rinv = act + C;
+    const T *row = rows + t * tok_stride;
+    if (conv_w) {
+        const ConvTail tail(state, slot_stride, tail_off, tok_pos, tok_start, tok_state, tok_seq, num_tokens, C, taps, t);
+        bool wide = false;
+        if constexpr (sizeof(T) == 2) {
+            wide = ConvTail::wide_ok(rows, tok_stride, conv_w, state, slot_stride, tail_off, C) &&
+                   (reinterpret_cast<uintptr_t>(bias) & 15) == 0;
+            if (wide) {
+                for (int c = threadIdx.x * 8; c < C; c += kRkThreads * 8) {
+                    const vec8_t<T> x = load8(row + c);
+                    float cur[8], b[8], a[8];
+#pragma unroll
+                    for (int j = 0; j < 8; ++j) {
+                        cur[j] = to_f(x[j]);
+                        b[j] = bias ? bias[c + j] : 0.f;
+                        a[j] = 0.f;
+                    }
+                    for (int k = taps - 1; k >= 1; --k) {       // inputs before the sequence are zero, biases included
+                        if (pos - k < 0) continue;
+                        float v[8];
+                        tail.at8(rows, tok_stride, c, pos - k, v);
+                        const float *wk = conv_w + static_cast<int64_t>(taps - 1 - k) * C + c;
+#pragma unroll
+                        for (int j = 0; j < 8; ++j) a[j] += wk[j] * (v[j] + b[j]);
+                    }
+                    const float *wl = conv_w + static_cast<int64_t>(taps - 1) * C + c;
+#pragma unroll
+                    for (int j = 0; j < 8; ++j) act[c + j] = a[j] + wl[j] * (cur[j] + b[j]);
+                    tail.save8(rows, tok_stride, c, cur);
+                }
+            }
+        }
+        for (int c = threadIdx.x; c < C && !wide; c += kRkThreads) {
+            const float cur = to_f(row[c]), b = bias ? bias[c] : 0.f;
+            float a = 0.f;
+            for (int k = taps - 1; k >= 1; --k)
+                if (pos - k >= 0)
+                    a += conv_w[static_cast<int64_t>(taps - 1 - k) * C + c] * (tail.at(rows, tok_stride, c, pos - k) + b);
+            act[c] = a + conv_w[static_cast<int64_t>(taps - 1) * C + c] * (cur + b);
+            tail.save(rows, tok_stride, c, cur);
+        }
+    } else {
+        bool wide = false;
+        if constexpr (sizeof(T) == 2) {
+            wide = (C & 7) == 0 && (tok_stride & 7) == 0 && (reinterpret_cast<uintptr_t>(rows) & 15) == 0;
+            if (wide) {
+                for (int c = threadIdx.x * 8; c < C; c += kRkThreads * 8) {
+                    const vec8_t<T> x = load8(row + c);
+#pragma unroll
+                    for (int j = 0; j < 8; ++j) act[c + j] = to_f(x[j]) + (bias ? bias[c + j] : 0.f);
+                }
+            }
+        }
+        for (int c = threadIdx.x; c < C && !wide; c += kRkThreads) act[c] = to_f(row[c]) + (bias ? bias[c] : 0.f);
+    }
+    rk_angles(cs, sn, freq, pos, pairs, rot_mult);
+    __syncthreads();
+    if (q_w) {
+        for (int h = wave; h < heads; h += kRkThreads / 64) {
+            float ss = 0.f;
+            for (int e = lane; e < d; e += 64) ss += act[h * d + e] * act[h * d + e];
+            ss = wave_allreduce_sum(ss);
+            if (lane == 0) rinv[h] = 1.0f / sqrtf(ss / static_cast<float>(d) + eps);
+        }
+        __syncthreads();
+    }
+    auto element = [&](int h, int e) {      // element e of head h: normed and rotated
+        const float *a = act + h * d, *w = h < nq ? q_w : k_w;
+        const float r = q_w ? rinv[h] : 1.f;
+        float n = q_w ? a[e] * r * w[e] : a[e];
+        if (e < rot_dims) {
+            const bool first = half ? e < pairs : (e & 1) == 0;
+            const int p = half ? (first ? e + pairs : e - pairs) : e ^ 1, i = half ? (first ? e : p) : e >> 1;
+            const float o = q_w ? a[p] * r * w[p] : a[p];
+            n = first ? n * cs[i] - o * sn[i] : n * cs[i] + o * sn[i];
+        }
+        return n;
+    };
+    const bool store = k_cache != nullptr;
+    int64_t blk = 0;
+    if (store) blk = block_table[static_cast<int64_t>(tok_seq[t]) * max_blocks_per_seq + pos / kRkBlock];
+    const int off = pos % kRkBlock;
+    T *qrow = q_out + t * q_out_stride;
+    T *kpage = k_cache + blk * block_stride, *vpage = v_cache + blk * block_stride;
+    const int outs = store ? heads : nq;
+    if (sizeof(T) == 2 && (k_dim & 7) == 0 && (q_out_stride & 7) == 0 && (block_stride & 7) == 0 &&
+        ((reinterpret_cast<uintptr_t>(q_out) | reinterpret_cast<uintptr_t>(k_cache)) & 15) == 0) {
+        const int per = k_dim >> 3;
+        for (int i = threadIdx.x; i < outs * per; i += kRkThreads) {
+            const int h = i / per, e0 = (i - h * per) * 8;
+            vec8_t<T> o;
+#pragma unroll
+            for (int j = 0; j < 8; ++j) o[j] = to_t<T>(e0 + j < d ? element(h, e0 + j) : 0.f);
+            store8(h < nq ? qrow + static_cast<int64_t>(h) * k_dim + e0
+                          : kpage + (static_cast<int64_t>(h - nq) * kRkBlock + off) * k_dim + e0, o);
+        }
+    } else {
+        for (int i = threadIdx.x; i < outs * k_dim; i += kRkThreads) {
+            const int h = i / k_dim, e = i - h * k_dim;
+            T *dst = h < nq ? qrow + static_cast<int64_t>(h) * k_dim : kpage + (static_cast<int64_t>(h - nq) * kRkBlock + off) * k_dim;
+            dst[e] = to_t<T>(e < d ? element(h, e) : 0.f);
+        }
+    }
+    if (!store) return;
+    for (int i = threadIdx.x; i < nk * v_dim; i += kRkThreads) {        // (the transposed page: 16 tokens of a column together)
+        const int g = i / v_dim, c = i - g * v_dim;
+        vpage[static_cast<int64_t>(i) * kRkBlock + off] = to_t<T>(c < dv ? act[heads * d + g * dv + c] * v_mult : 0.f);
+    }
+}
+
+template <typename T>
 __global__ __launch_bounds__(kRkThreads) void latent_rope_store_kv_kernel(
     const T *proj, T *qa, const double *freq, const float *c_w, T *k_cache, T *v_cache, const int32_t *block_table,
     const int32_t *tok_seq, const int32_t *tok_pos, int H, int d, int dr, int r, int64_t proj_stride, int64_t dkv_col,
@@ -410,6 +539,35 @@ extern "C" int swl_qk_norm_rope_store_kv(const void *rows, void *q_out, const fl
                            q_w, k_w, q_mult, freq, static_cast<T *>(k_cache), static_cast<T *>(v_cache), block_table, tok_seq,
                            tok_pos, num_q_heads, num_k_heads, num_v_heads, dim, vdim, rot_dims, half, rot_mult, tok_stride,
                            q_out_stride, k_dim, v_dim, keys_as_values, max_blocks_per_seq, block_stride, eps);
+    });
+    return swl::check_launch();
+}
+
+extern "C" int swl_qkv_conv_rope_store_kv(
+    const void *rows, int64_t tok_stride, void *q_out, int64_t q_out_stride, const float *bias, const float *conv_w, int32_t taps,
+    const float *q_w, const float *k_w, const double *freq, int32_t rot_dims, int32_t half, double rot_mult, float v_mult,
+    void *k_cache, void *v_cache, const int32_t *block_table, int32_t max_blocks_per_seq, int64_t block_stride, float *state,
+    int64_t slot_stride, int64_t tail_off, const int32_t *tok_pos, const int32_t *tok_start, const int32_t *tok_state,
+    const int32_t *tok_seq, int64_t num_tokens, int32_t num_q_heads, int32_t num_kv_heads, int32_t dim, int32_t vdim, int32_t k_dim,
+    int32_t v_dim, float eps, int32_t dtype, swl_stream_t stream) {
+    if (num_tokens < 0 || num_q_heads <= 0 || num_kv_heads <= 0 || dim <= 0 || vdim <= 0) return SWL_ERR_BAD_ARG;
+    if (rot_dims < 0 || (rot_dims & 1) || rot_dims > dim || (!half && (dim & 1))) return SWL_ERR_BAD_ARG;
+    if (k_dim < dim || v_dim < vdim || q_out_stride < static_cast<int64_t>(num_q_heads) * k_dim) return SWL_ERR_BAD_ARG;
+    const int64_t C = static_cast<int64_t>(num_q_heads + num_kv_heads) * dim + static_cast<int64_t>(num_kv_heads) * vdim;
+    if (tok_stride < C || (conv_w && taps < 1) || (!q_w) != (!k_w)) return SWL_ERR_BAD_ARG;
+    if (num_tokens == 0) return SWL_OK;
+    if (!rows || !q_out || rows == q_out || !tok_pos || !tok_seq || (rot_dims > 0 && !freq)) return SWL_ERR_BAD_ARG;
+    if (conv_w && (!tok_start || (taps > 1 && (!state || !tok_state)))) return SWL_ERR_BAD_ARG;
+    if (k_cache && (!v_cache || !block_table || max_blocks_per_seq <= 0)) return SWL_ERR_BAD_ARG;
+    const size_t lds = (static_cast<size_t>(C) + num_q_heads + num_kv_heads) * sizeof(float);
+    if (num_tokens > 0x7fffffffLL || rot_dims > 2 * swl::kRkMaxPairs || lds > 60 * 1024) return SWL_ERR_UNSUPPORTED;
+    SWL_DISPATCH_DTYPE3(dtype, T, {
+        hipLaunchKernelGGL((swl::qkv_conv_rope_store_kv_kernel<T>), dim3(static_cast<unsigned>(num_tokens)), dim3(swl::kRkThreads),
+                           lds, static_cast<hipStream_t>(stream), static_cast<const T *>(rows), tok_stride, static_cast<T *>(q_out),
+                           q_out_stride, bias, conv_w, taps, q_w, k_w, freq, rot_dims, half, rot_mult, v_mult,
+                           static_cast<T *>(k_cache), static_cast<T *>(v_cache), block_table, max_blocks_per_seq, block_stride,
+                           state, slot_stride, tail_off, tok_pos, tok_start, tok_state, tok_seq, num_tokens, num_q_heads,
+                           num_kv_heads, dim, vdim, k_dim, v_dim, eps);
     });
     return swl::check_launch();
 }

@@ -215,7 +215,7 @@ __global__ __launch_bounds__(1024) void ssd_scan_kernel(float *y, const float *x
 template <typename T>
 __global__ __launch_bounds__(kSsThreads) void gated_group_rmsnorm_kernel(T *out, const float *y, const T *gate,
                                                                          int64_t gate_stride, const float *w, float eps,
-                                                                         int cols, int part) {
+                                                                         int cols, int part, int64_t out_stride) {
     __shared__ float red[kSsThreads / 64];
     const int64_t t = blockIdx.x;
     const int c0 = blockIdx.y * part;
@@ -236,7 +236,7 @@ __global__ __launch_bounds__(kSsThreads) void gated_group_rmsnorm_kernel(T *out,
     for (int c = threadIdx.x; c < part; c += kSsThreads) {
         const float z = to_f(gate[t * gate_stride + c0 + c]);
         const float v = y[t * cols + c0 + c] * (z * ss_sigmoid(z));
-        out[t * cols + c0 + c] = to_t<T>(v * r * w[c0 + c]);
+        out[t * out_stride + c0 + c] = to_t<T>(v * r * w[c0 + c]);
     }
 }
 
@@ -328,17 +328,17 @@ extern "C" int swl_ssd_scan(float *y, const float *xbc, const float *dt, const f
     return SWL_ERR_UNSUPPORTED;
 }
 
-extern "C" int swl_gated_group_rmsnorm(void *out, const float *y, const void *gate, int64_t gate_stride, const float *w,
-                                       float eps, int64_t num_tokens, int32_t cols, int32_t groups, int32_t dtype,
+extern "C" int swl_gated_group_rmsnorm(void *out, int64_t out_stride, const float *y, const void *gate, int64_t gate_stride,
+                                       const float *w, float eps, int64_t num_tokens, int32_t cols, int32_t groups, int32_t dtype,
                                        swl_stream_t stream) {
-    if (num_tokens < 0 || cols <= 0 || groups <= 0 || cols % groups || gate_stride < cols) return SWL_ERR_BAD_ARG;
+    if (num_tokens < 0 || cols <= 0 || groups <= 0 || cols % groups || gate_stride < cols || out_stride < cols) return SWL_ERR_BAD_ARG;
     if (num_tokens == 0) return SWL_OK;
     if (!out || !y || !gate || !w) return SWL_ERR_BAD_ARG;
     if (num_tokens > 0x7fffffffLL || groups > 65535) return SWL_ERR_UNSUPPORTED;
     SWL_DISPATCH_DTYPE3(dtype, T, {
         hipLaunchKernelGGL((swl::gated_group_rmsnorm_kernel<T>), dim3(static_cast<unsigned>(num_tokens), groups),
                            dim3(swl::kSsThreads), 0, static_cast<hipStream_t>(stream), static_cast<T *>(out), y,
-                           static_cast<const T *>(gate), gate_stride, w, eps, cols, cols / groups);
+                           static_cast<const T *>(gate), gate_stride, w, eps, cols, cols / groups, out_stride);
     });
     return swl::check_launch();
 }

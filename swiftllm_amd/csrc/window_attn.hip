@@ -19,6 +19,9 @@
 //   * num_v_heads < num_kv_heads: several key heads share one value head (value head = key head % num_v_heads) — two
 //     score maps over the same values, laid out map-major, are 2 G key heads over G value heads;
 //   * out_f32: the result leaves in fp32 (for a combination of maps that cancels);
+//   * slopes[H]: slope times the distance (query position - key position) is taken off the (capped) score;
+//   * out_dim / out_stride: pages may hold values wider than the heads are (vdim columns, of which the first out_dim count) and the
+//     result may be a column slice of wider rows; gate: the result is multiplied by sigmoid(gate[t][h * out_dim + c]);
 //   * without a mixing matrix the heads are independent: more than 32 of them (or more than the accumulators and the LDS of
 //     one workgroup hold) are shared out over blockIdx.y, every workgroup taking a group of consecutive heads.
 #include "swl_common.h"
@@ -42,7 +45,8 @@ __global__ __launch_bounds__(kWaThreads) void window_attn_kernel(
     T *out, const T *q, const T *k_cache, const T *v_cache, const int32_t *block_table, const int32_t *tok_seq,
     const int32_t *tok_pos, const float *talk, const float *rel, int rel_len, int H, int G, int d, int dv,
     int64_t q_tok_stride, int window, float scale, float softcap, int max_blocks_per_seq, int64_t block_stride,
-    int mask_kind, const float *sink, int GV, int out_f32, int Hall) {
+    int mask_kind, const float *sink, int GV, int out_f32, int Hall, const float *slopes, int out_dim, int64_t out_stride,
+    const T *gate, int64_t gate_stride) {
     // H: heads of this workgroup, starting at head hb of the token's Hall heads (G: key heads per Hall query heads)
     extern __shared__ float lds[];
     float *qf = lds;                        // [H * d]
@@ -64,6 +68,7 @@ __global__ __launch_bounds__(kWaThreads) void window_attn_kernel(
     if (hb + H > Hall) H = Hall - hb;
     if (sink) sink += hb;
     if (rel) rel += static_cast<int64_t>(hb) * rel_len;
+    if (slopes) slopes += hb;
 
     const T *qrow = q + t * q_tok_stride + static_cast<int64_t>(hb) * d;
     for (int i = tid; i < H * d; i += kWaThreads) qf[i] = to_f(qrow[i]);
@@ -121,6 +126,7 @@ __global__ __launch_bounds__(kWaThreads) void window_attn_kernel(
                 }
                 // learned bias by distance (query position - key position), one row of the table per head
                 if (rel) a += rel[static_cast<int64_t>(h) * rel_len + min(nkeys - 1 - (c0 + lane), rel_len - 1)];
+                if (slopes) a -= slopes[h] * static_cast<float>(nkeys - 1 - (c0 + lane));
                 mixed = a;
             }
             const float cmax = wave_allreduce_max(mixed);
@@ -168,15 +174,18 @@ __global__ __launch_bounds__(kWaThreads) void window_attn_kernel(
         if (lane == 0) alpha[h] = al / l;
     }
     __syncthreads();
-    const int64_t obase = (t * static_cast<int64_t>(Hall) + hb) * dv;
 #pragma unroll
     for (int i = 0; i < kWaMaxAcc; ++i) {
         if (i >= nacc) break;
         const int idx = tid + i * kWaThreads;
         if (idx < H * dv) {
-            const float o = acc[i] * alpha[idx / dv];
-            if (out_f32) reinterpret_cast<float *>(out)[obase + idx] = o;
-            else out[obase + idx] = to_t<T>(o);
+            const int h = idx / dv, c = idx - h * dv;
+            if (c >= out_dim) continue;
+            float o = acc[i] * alpha[h];
+            const int64_t hc = static_cast<int64_t>(hb + h) * out_dim + c;
+            if (gate) o /= 1.0f + expf(-to_f(gate[t * gate_stride + hc]));
+            if (out_f32) reinterpret_cast<float *>(out)[t * out_stride + hc] = o;
+            else out[t * out_stride + hc] = to_t<T>(o);
         }
     }
 }
@@ -193,12 +202,15 @@ extern "C" int swl_masked_attn(void *out, const void *q, const void *k_cache, co
                                int32_t num_q_heads, int32_t num_kv_heads,
                                int32_t dim, int32_t vdim, int64_t q_tok_stride, int32_t window, float scale,
                                float softcap, int32_t max_blocks_per_seq, int64_t block_stride, int32_t mask_kind,
-                               const float *sink, int32_t num_v_heads, int32_t out_f32, int32_t dtype,
+                               const float *sink, int32_t num_v_heads, int32_t out_f32, const float *slopes,
+                               int32_t out_dim, int64_t out_stride, const void *gate, int64_t gate_stride, int32_t dtype,
                                swl_stream_t stream) {
     if (num_tokens < 0 || num_q_heads <= 0 || num_kv_heads <= 0 || dim <= 0 || vdim <= 0 || window < 0)
         return SWL_ERR_BAD_ARG;
     if (num_q_heads % num_kv_heads) return SWL_ERR_BAD_ARG;
     if (mask_kind < 0 || mask_kind > 1 || num_v_heads <= 0 || num_kv_heads % num_v_heads) return SWL_ERR_BAD_ARG;
+    if (out_dim <= 0 || out_dim > vdim || out_stride < static_cast<int64_t>(num_q_heads) * out_dim) return SWL_ERR_BAD_ARG;
+    if (gate && gate_stride < static_cast<int64_t>(num_q_heads) * out_dim) return SWL_ERR_BAD_ARG;
     if (num_tokens == 0) return SWL_OK;
     if (!out || !q || !k_cache || !v_cache || !block_table || !tok_seq || !tok_pos || (rel && rel_len <= 0))
         return SWL_ERR_BAD_ARG;
@@ -222,7 +234,8 @@ extern "C" int swl_masked_attn(void *out, const void *q, const void *k_cache, co
                            static_cast<const T *>(k_cache), static_cast<const T *>(v_cache), block_table, tok_seq,
                            tok_pos, talk, rel, rel_len, hpg, num_kv_heads, dim, vdim, q_tok_stride, window, scale,
                            softcap,
-                           max_blocks_per_seq, block_stride, mask_kind, sink, num_v_heads, out_f32, num_q_heads);
+                           max_blocks_per_seq, block_stride, mask_kind, sink, num_v_heads, out_f32, num_q_heads, slopes, out_dim, out_stride,
+                           static_cast<const T *>(gate), gate_stride);
     });
     return swl::check_launch();
 }
@@ -236,5 +249,6 @@ extern "C" int swl_window_attn(void *out, const void *q, const void *k_cache, co
                                swl_stream_t stream) {
     return swl_masked_attn(out, q, k_cache, v_cache, block_table, tok_seq, tok_pos, talk, rel, rel_len, num_tokens,
                            num_q_heads, num_kv_heads, dim, vdim, q_tok_stride, window, scale, softcap, max_blocks_per_seq,
-                           block_stride, 0, nullptr, num_kv_heads > 0 ? num_kv_heads : 1, 0, dtype, stream);
+                           block_stride, 0, nullptr, num_kv_heads > 0 ? num_kv_heads : 1, 0, nullptr, vdim,
+                           static_cast<int64_t>(num_q_heads) * vdim, nullptr, 0, dtype, stream);
 }

@@ -14,7 +14,8 @@
 //
 // The general entry point (swl_masked_attn_tiles) adds: mask_kind 1 (chunked visibility: keys [floor(p / window) * window, p]),
 // sink[H] (a logit per head that joins the denominator only), num_v_heads (value head = key head % num_v_heads: score maps
-// that share their values), out_f32 (fp32 result), and a split of the heads over blockIdx.z (head_groups: every group of
+// that share their values), out_f32 (fp32 result), slopes[H] (slope x distance off the capped score), out_dim / out_stride / gate (the
+// first out_dim of the DV value columns, into a column slice of wider rows, times the sigmoid of a gate element), and a split of the heads over blockIdx.z (head_groups: every group of
 // heads_per_group heads is a workgroup of its own — many heads over one shared key head, wide value heads).
 //
 // HEADS mode (decode steps of a layer whose heads all read ONE key head, e.g. latent attention): a tile is one token and the
@@ -37,7 +38,7 @@ __global__ __launch_bounds__(NW * 64, (HPW <= 2 && NW == 4 && HPW * (D + DV) <= 
     const float *__restrict__ rel, int rel_len, int H, int G,
     int64_t q_tok_stride, int window, float scale, float softcap, int max_blocks_per_seq, int64_t block_stride,
     float *part_o, float *part_ml, int64_t num_tokens, int nbuf, int mask_kind, const float *__restrict__ sink, int GV,
-    int out_f32, int hpg) {
+    int out_f32, int hpg, const float *__restrict__ slopes, int out_dim, int64_t out_stride, const T *gate, int64_t gate_stride) {
     // [nbuf][H][64 lanes][4] capped scores of a page, then [H][H] the mixing matrix. nbuf = 2: pages alternate between two
     // score buffers and ONE barrier per page suffices (a wave that is a page ahead writes the other buffer)
     extern __shared__ float s_all[];
@@ -217,6 +218,15 @@ __global__ __launch_bounds__(NW * 64, (HPW <= 2 && NW == 4 && HPW * (D + DV) <= 
                     mixed[hh][r] += rh[min(max(qpos - (kpos0 + r), 0), rel_len - 1)] * kLog2e;
             }
         }
+        if (slopes) {       // (base-2 units, as the scores)
+            const float d0 = static_cast<float>(qpos - kpos0) * kLog2e;
+#pragma unroll
+            for (int hh = 0; hh < HPW; ++hh) {
+                const float sl = slopes[HEADS ? (qok ? hbase + li : hbase) : min(h0 + hh, H - 1)];
+#pragma unroll
+                for (int r = 0; r < 4; ++r) mixed[hh][r] = fmaf(sl, r * kLog2e - d0, mixed[hh][r]);
+            }
+        }
 #pragma unroll
         for (int hh = 0; hh < HPW; ++hh) {
             const int h = h0 + hh;
@@ -294,9 +304,20 @@ __global__ __launch_bounds__(NW * 64, (HPW <= 2 && NW == 4 && HPW * (D + DV) <= 
             for (int ct = 0; ct < CT; ++ct) {
                 float4_t o = acc[hh][ct];
                 mfma_results_ready<4>(o);
-                if (qok) {
-                    const int64_t at = (static_cast<int64_t>(orow) * H + ohead) * DV + ct * 16 + 4 * lq;
-                    if (out_f32) {
+                const int c = ct * 16 + 4 * lq;
+                if (qok && c < out_dim) {
+                    const int64_t hc = static_cast<int64_t>(ohead) * out_dim + c, at = orow * out_stride + hc;
+                    if (gate || (out_dim & 3)) {        // (uniform) element by element
+#pragma unroll
+                        for (int r = 0; r < 4; ++r) {
+                            if (c + r < out_dim) {
+                                float v = o[r] * inv;
+                                if (gate) v /= 1.0f + fast_exp2(-kLog2e * to_f(gate[orow * gate_stride + hc + r]));
+                                if (out_f32) reinterpret_cast<float *>(out)[at + r] = v;
+                                else out[at + r] = to_t<T>(v);
+                            }
+                        }
+                    } else if (out_f32) {
 #pragma unroll
                         for (int r = 0; r < 4; ++r) o[r] *= inv;
                         *reinterpret_cast<float4_t *>(reinterpret_cast<float *>(out) + at) = o;
@@ -318,7 +339,8 @@ __global__ __launch_bounds__(NW * 64, (HPW <= 2 && NW == 4 && HPW * (D + DV) <= 
 template <typename T>
 __global__ __launch_bounds__(256) void window_attn_combine_kernel(T *out, const float *part_o, const float *part_ml,
                                                                   int64_t rows, int dv, int nsplit, const float *sink, int H,
-                                                                  int out_f32) {
+                                                                  int out_f32, int out_dim, int64_t out_stride, const T *gate,
+                                                                  int64_t gate_stride) {
     __shared__ float wgt[64];
     __shared__ float inv_den;
     const int64_t row = blockIdx.x;     // (token, head)
@@ -341,11 +363,14 @@ __global__ __launch_bounds__(256) void window_attn_combine_kernel(T *out, const 
     }
     __syncthreads();
     const float inv = inv_den;
-    for (int c = threadIdx.x; c < dv; c += blockDim.x) {
+    const int64_t tok = row / H, hc0 = (row - tok * H) * out_dim;
+    for (int c = threadIdx.x; c < out_dim; c += blockDim.x) {
         float a = 0.f;
         for (int s = 0; s < nsplit; ++s) a += wgt[s] * part_o[(s * rows + row) * dv + c];
-        if (out_f32) reinterpret_cast<float *>(out)[row * dv + c] = a * inv;
-        else out[row * dv + c] = to_t<T>(a * inv);
+        a *= inv;
+        if (gate) a /= 1.0f + expf(-to_f(gate[tok * gate_stride + hc0 + c]));
+        if (out_f32) reinterpret_cast<float *>(out)[tok * out_stride + hc0 + c] = a;
+        else out[tok * out_stride + hc0 + c] = to_t<T>(a);
     }
 }
 
@@ -355,22 +380,22 @@ int launch_wm(int hpw, dim3 grid, size_t lds, hipStream_t s, T *out, const T *q,
               const float *talk, const float *rel, int rel_len, int H, int G, int64_t qs, int window, float scale,
               float softcap, int mb, int64_t bs,
               float *po, float *pml, int64_t nt, int nbuf, int mask_kind, const float *sink, int GV, int out_f32, int hpg,
-              bool heads_mode) {
+              bool heads_mode, const float *slopes, int od, int64_t ostr, const T *gate, int64_t gstr) {
     if (heads_mode) {       // rows are heads: one wave per workgroup, grid.z = groups of sixteen heads
         hipLaunchKernelGGL((window_attn_mfma_kernel<T, D, DV, 1, 1, false, true>), grid, dim3(64), 0, s, out, q, kc, vc, bt, ts,
                            tp, r0, cn, nullptr, nullptr, 0, H, G, qs, window, scale, softcap, mb, bs, po, pml, nt, nbuf,
-                           mask_kind, sink, GV, out_f32, hpg);
+                           mask_kind, sink, GV, out_f32, hpg, slopes, od, ostr, gate, gstr);
         if (grid.y > 1) {
             const int64_t rows = nt * H;
             hipLaunchKernelGGL((window_attn_combine_kernel<T>), dim3(static_cast<unsigned>(rows)), dim3(DV < 256 ? 64 : 256), 0,
-                               s, out, po, pml, rows, DV, static_cast<int>(grid.y), sink, H, out_f32);
+                               s, out, po, pml, rows, DV, static_cast<int>(grid.y), sink, H, out_f32, od, ostr, gate, gstr);
         }
         return check_launch();
     }
 #define SWL_WM_LAUNCH1(HPW, NW, MIX)                                                                                         \
     hipLaunchKernelGGL((window_attn_mfma_kernel<T, D, DV, HPW, NW, MIX>), grid, dim3(NW * 64), MIX ? lds : 0, s, out, q, kc, \
                        vc, bt, ts, tp, r0, cn, talk, rel, rel_len, H, G, qs, window, scale, softcap, mb, bs, po, pml, nt, nbuf, mask_kind,  \
-                       sink, GV, out_f32, hpg)
+                       sink, GV, out_f32, hpg, slopes, od, ostr, gate, gstr)
     // (a wave's accumulators: HPW * DV / 4 registers — variants beyond 128 of them are not compiled for the wide shapes)
 #define SWL_WM_LAUNCH(HPW, NW)                                 \
     if constexpr (!MIXOK && HPW * DV > 512) {                  \
@@ -393,7 +418,7 @@ int launch_wm(int hpw, dim3 grid, size_t lds, hipStream_t s, T *out, const T *q,
     if (grid.y > 1) {
         const int64_t rows = nt * H;
         hipLaunchKernelGGL((window_attn_combine_kernel<T>), dim3(static_cast<unsigned>(rows)), dim3(DV < 256 ? 64 : 256), 0, s,
-                           out, po, pml, rows, DV, static_cast<int>(grid.y), sink, H, out_f32);
+                           out, po, pml, rows, DV, static_cast<int>(grid.y), sink, H, out_f32, od, ostr, gate, gstr);
     }
     return check_launch();
 }
@@ -441,12 +466,16 @@ extern "C" int swl_masked_attn_tiles(void *out, const void *q, const void *k_cac
                                      int32_t vdim, int64_t q_tok_stride, int32_t window, float scale, float softcap,
                                      int32_t max_blocks_per_seq, int64_t block_stride, int32_t key_splits,
                                      float *scratch, int64_t num_tokens, int32_t mask_kind, const float *sink,
-                                     int32_t num_v_heads, int32_t out_f32, int32_t heads_per_group, int32_t dtype,
+                                     int32_t num_v_heads, int32_t out_f32, int32_t heads_per_group, const float *slopes,
+                                     int32_t out_dim, int64_t out_stride, const void *gate, int64_t gate_stride, int32_t dtype,
                                      swl_stream_t stream) {
     if (num_tiles < 0 || window < 0 || key_splits < 1 || key_splits > 64) return SWL_ERR_BAD_ARG;
     if (key_splits > 1 && (!scratch || num_tokens <= 0 || (reinterpret_cast<uintptr_t>(scratch) & 15)))
         return SWL_ERR_BAD_ARG;
     if (mask_kind < 0 || mask_kind > 1 || heads_per_group < -1) return SWL_ERR_BAD_ARG;
+    if (out_dim <= 0 || out_dim > vdim || out_stride < static_cast<int64_t>(num_q_heads) * out_dim) return SWL_ERR_BAD_ARG;
+    if (gate && gate_stride < static_cast<int64_t>(num_q_heads) * out_dim) return SWL_ERR_BAD_ARG;
+    if (!gate && out_dim % 4 == 0 && (out_stride & 3)) return SWL_ERR_BAD_ARG;      // (4-element stores)
     // heads_per_group -1: the rows of a tile are heads (every tile is ONE token, all heads read one key head, no mix, no bias)
     const bool heads_mode = heads_per_group == -1;
     if (heads_mode && (talk || rel || num_kv_heads != 1 || num_tiles != num_tokens)) return SWL_ERR_BAD_ARG;
@@ -489,7 +518,8 @@ extern "C" int swl_masked_attn_tiles(void *out, const void *q, const void *k_cac
                                           static_cast<const T *>(k_cache), static_cast<const T *>(v_cache), block_table, \
                                           tok_seq, tok_pos, tile_row0, tile_cnt, talk, rel, rel_len, num_q_heads, num_kv_heads, \
                                           q_tok_stride, window, scale, softcap, max_blocks_per_seq, block_stride, part_o, \
-                                          part_ml, num_tokens, nbuf, mask_kind, sink, num_v_heads, out_f32, hpg, heads_mode);
+                                          part_ml, num_tokens, nbuf, mask_kind, sink, num_v_heads, out_f32, hpg, heads_mode, slopes, out_dim, out_stride, \
+                                          static_cast<const T *>(gate), gate_stride);
 #define SWL_WM_SHAPE_MIX(DD, DDV) SWL_WM_SHAPE_(DD, DDV, true)
 #define SWL_WM_SHAPE_PLAIN(DD, DDV) SWL_WM_SHAPE_(DD, DDV, false)
     SWL_DISPATCH_DTYPE(dtype, T, {
@@ -513,5 +543,6 @@ extern "C" int swl_window_attn_tiles(void *out, const void *q, const void *k_cac
     return swl_masked_attn_tiles(out, q, k_cache, v_cache, block_table, tok_seq, tok_pos, tile_row0, tile_cnt, talk, rel,
                                  rel_len, num_tiles, num_q_heads, num_kv_heads, dim, vdim, q_tok_stride, window, scale,
                                  softcap, max_blocks_per_seq, block_stride, key_splits, scratch, num_tokens, 0, nullptr,
-                                 num_kv_heads, 0, 0, dtype, stream);
+                                 num_kv_heads, 0, 0, nullptr, vdim, static_cast<int64_t>(num_q_heads) * vdim, nullptr, 0, dtype,
+                                 stream);
 }

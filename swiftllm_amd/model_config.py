@@ -858,3 +858,175 @@ class RokevikModelConfig:
     def load_from_model_path(model_path: str) -> "RokevikModelConfig":
         with open(os.path.join(model_path, "config.json"), "r", encoding="utf-8") as f:
             return RokevikModelConfig(json.load(f))
+
+
+# ---- Vafozen ---------------------------------------------------------------------------------------------------------------
+class VafozenAttentionConfig:
+    """Softmax attention with biased projections, the left half of a side-by-side mixer. `convolved` = False: weighted q/k norm, no
+    rotation, a distance penalty per head (slope_h = 2^(-8 (h + 1) / heads)), keys of the query's own chunk of `chunk` positions
+    (0: every earlier key). `convolved` = True: causal convolutions of `conv_taps` taps on q, k and v (0: none), rotate-half
+    rotary, tanh soft-capping (0: none) and an element-wise output gate; every earlier key."""
+    kind = "attention"
+
+    def __init__(self, mixer: dict, convolved: bool):
+        self.convolved = convolved
+        self.num_q_heads = int(mixer["heads"])
+        self.num_kv_heads = int(mixer.get("kv_heads", self.num_q_heads))
+        self.head_dim = int(mixer["dim"])
+        self.value_dim = int(mixer.get("vdim", self.head_dim))
+        self.scale = float(mixer["scale"])
+        mask = mixer.get("mask") or {}
+        cap = mixer.get("softcap")
+        self.chunk = int(mask["size"]) if mask.get("size") and not convolved else 0
+        self.conv_taps = int(mixer.get("conv") or 0) if convolved else 0
+        self.softcap = float(cap) if cap and convolved else 0.0
+        self.rot = RotaryConfig(mixer.get("rot") if convolved else None, self.head_dim, half=True)
+        if self.num_q_heads % self.num_kv_heads:
+            raise ValueError(f"heads ({self.num_q_heads}) must be a multiple of kv_heads ({self.num_kv_heads})")
+        if self.chunk < 0 or self.conv_taps < 0:
+            raise ValueError(f"bad mask size ({self.chunk}) or conv ({self.conv_taps})")
+
+    def slopes(self):
+        """The distance penalty of every head, or None."""
+        if self.convolved:
+            return None
+        return [2.0 ** (-8.0 * (h + 1) / self.num_q_heads) for h in range(self.num_q_heads)]
+
+    @property
+    def q_size(self) -> int:
+        return self.num_q_heads * self.head_dim
+
+    @property
+    def k_size(self) -> int:
+        return self.num_kv_heads * self.head_dim
+
+    @property
+    def v_size(self) -> int:
+        return self.num_kv_heads * self.value_dim
+
+    @property
+    def channels(self) -> int:
+        """Rows of the fused q | k | v projection (what the convolutions run over)."""
+        return self.q_size + self.k_size + self.v_size
+
+    @property
+    def o_size(self) -> int:
+        return self.num_q_heads * self.value_dim
+
+
+class LinearAttentionConfig:
+    """Gated linear attention: a state [dim, vdim] per head, a decay sigmoid(.)^(1 / tau) per key channel."""
+    kind = "linear_attention"
+
+    def __init__(self, mixer: dict):
+        self.num_heads = int(mixer["heads"])
+        self.key_dim = int(mixer["dim"])
+        self.value_dim = int(mixer.get("vdim", self.key_dim))
+        self.tau = float(mixer["tau"])
+        if self.tau <= 0:
+            raise ValueError(f"tau ({self.tau}) must be positive")
+
+    @property
+    def keys(self) -> int:
+        return self.num_heads * self.key_dim
+
+    @property
+    def inner(self) -> int:
+        return self.num_heads * self.value_dim
+
+    @property
+    def state_elems(self) -> int:
+        return self.num_heads * self.key_dim * self.value_dim
+
+
+class TimeMixingConfig:
+    """Time mixing of token-shifted inputs: a state [dim, dim] per head, a decay per key channel, a bonus for the current token."""
+    kind = "time_mixing"
+
+    def __init__(self, mixer: dict):
+        self.num_heads = int(mixer["heads"])
+        self.key_dim = self.value_dim = int(mixer["dim"])
+
+    @property
+    def inner(self) -> int:
+        return self.num_heads * self.value_dim
+
+    keys = inner
+
+    @property
+    def state_elems(self) -> int:
+        return self.num_heads * self.key_dim * self.value_dim
+
+
+class VafozenSideBySideConfig:
+    """Two mixers on the same input: left_scale * attention + right_scale * recurrence."""
+
+    def __init__(self, mixer: dict, kind: str):
+        self.kind = kind
+        self.left = VafozenAttentionConfig(mixer["left"], convolved=kind == "parallel_2")
+        self.right = (TimeMixingConfig if kind == "parallel_2" else LinearAttentionConfig)(mixer["right"])
+        self.left_scale = float(mixer.get("left_scale", 1.0))
+        self.right_scale = float(mixer.get("right_scale", 1.0))
+
+
+class VafozenMlpConfig:
+    """`dense`: down(silu(gate h) * up h)."""
+
+    def __init__(self, mlp: dict):
+        self.kind = mlp["kind"]
+        if self.kind != "dense":
+            raise ValueError(f"unsupported mlp.kind {self.kind!r}")
+        self.ffn_inter_dim = int(mlp["ff"])
+
+
+class VafozenLayerConfig:
+    def __init__(self, layer: dict):
+        self.type = layer["type"]
+        if self.type in ("parallel", "parallel_2"):
+            self.mixer = VafozenSideBySideConfig(layer["mixer"], self.type)
+        elif self.type == "mamba2":
+            self.mixer = StateSpaceConfig(layer["mixer"])
+        else:
+            raise ValueError(f"unsupported layer type {self.type!r}")
+        self.mlp = VafozenMlpConfig(layer["mlp"]) if layer.get("mlp") else None
+
+    @property
+    def attention(self) -> VafozenAttentionConfig:
+        """The layer's attention (whose keys and values the block pool holds), or None."""
+        return self.mixer.left if self.type != "mamba2" else None
+
+
+class VafozenModelConfig:
+    """Vafozen: a decoder-only model whose layers add mixer(h) + ff(h) of ONE normed input (RMS norm, weight stored around zero) to an
+    fp32 stream. Mixers, in any order: chunked distance-penalised attention beside gated linear attention, convolved rotary
+    attention beside time mixing, a state-space recurrence. Every size and constant is read from config.json. The design has no
+    position table: `max_positions`, if config.json gives it, bounds a sequence; otherwise the bound is DEFAULT_MAX_POSITIONS."""
+    DEFAULT_MAX_POSITIONS = 1 << 20
+
+    def __init__(self, model_config: dict):
+        if model_config.get("architecture") != "Vafozen":
+            raise AssertionError(f"unsupported architecture {model_config.get('architecture')!r}")
+        self.vocab_size = int(model_config["vocab"])
+        self.hidden_size = int(model_config["width"])
+        self.max_position_embeddings = int(model_config.get("max_positions") or self.DEFAULT_MAX_POSITIONS)
+        self.norm_eps = float(model_config["norm"]["eps"])
+        self.embedding_scale = float((model_config.get("embedding") or {}).get("scale", 1.0))
+        self.layers = [VafozenLayerConfig(layer) for layer in model_config["layers"]]
+        self.num_layers = len(self.layers)
+        attn = [l.attention for l in self.layers if l.attention is not None]
+        # what the scheduler-facing code reads off any model's configuration
+        self.num_q_heads = max((m.num_q_heads for m in attn), default=1)
+        self.num_kv_heads = max((m.num_kv_heads for m in attn), default=1)
+        self.head_dim = max((m.head_dim for m in attn), default=1)
+
+    def kv_elems_per_token(self) -> int:
+        """K and V elements one token occupies over the layers with an attention."""
+        return sum(l.attention.k_size + l.attention.v_size for l in self.layers if l.attention is not None)
+
+    def get_kvslot_size(self, dtype: torch.dtype = torch.bfloat16) -> int:
+        return max(self.kv_elems_per_token(), 1) * dtype.itemsize
+
+    @staticmethod
+    def load_from_model_path(model_path: str) -> "VafozenModelConfig":
+        with open(os.path.join(model_path, "config.json"), "r", encoding="utf-8") as f:
+            return VafozenModelConfig(json.load(f))

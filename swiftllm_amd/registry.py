@@ -16,6 +16,7 @@ MODELS = {
     "Rosilix": ("swiftllm_amd.model_config:RosilixModelConfig", "swiftllm_amd.worker.rosilix_model:RosilixModel"),
     "Ratilorn": ("swiftllm_amd.model_config:RatilornModelConfig", "swiftllm_amd.worker.ratilorn_model:RatilornModel"),
     "Rokevik": ("swiftllm_amd.model_config:RokevikModelConfig", "swiftllm_amd.worker.rokevik_model:RokevikModel"),
+    "Vafozen": ("swiftllm_amd.model_config:VafozenModelConfig", "swiftllm_amd.worker.vafozen_model:VafozenModel"),
 }
 
 

@@ -171,11 +171,12 @@ class StepPlan:
     chunk_row0: np.ndarray = None       # [NC] int32 first token row of each chunk
     chunk_cnt: np.ndarray = None        # [NC] int32 tokens in it
     seq_chunk0: np.ndarray = None       # [S] int32
+    seq_tile0: np.ndarray = None        # [S] int32 the first tile of each sequence
 
     TILE = 16
     CHUNK = 32
     SEGMENTS = ("input_ids", "tok_pos", "tok_seq", "want_rows", "tile_row0", "tile_cnt", "seq_row0", "seq_cnt", "tok_start",
-                "tok_state", "chunk_row0", "chunk_cnt", "seq_chunk0")
+                "tok_state", "chunk_row0", "chunk_cnt", "seq_chunk0", "seq_tile0")
 
     def packed_layout(self):
         out, off = [], 0
@@ -238,8 +239,10 @@ def plan_step(entries: Sequence[StepEntry], vocab_size: int = None, max_position
     counts = np.asarray([len(e.tokens) for e in entries], dtype=np.int32)
     starts = np.asarray([e.start for e in entries], dtype=np.int32)
     chunks = -(-counts // StepPlan.CHUNK)
+    seq_tiles = -(-counts // StepPlan.TILE)
     return StepPlan(tile_row0=tile_row0, tile_cnt=tile_cnt, seq_cnt=counts, chunk_row0=chunk_row0, chunk_cnt=chunk_cnt,
                     seq_chunk0=(np.cumsum(chunks) - chunks).astype(np.int32),
+                    seq_tile0=(np.cumsum(seq_tiles) - seq_tiles).astype(np.int32),
                     seq_row0=(np.cumsum(counts) - counts).astype(np.int32), tok_start=np.repeat(starts, counts),
                     tok_state=np.zeros(base, dtype=np.int32),
                     num_tokens=base, num_seqs=len(seq_ids), seq_ids_list=seq_ids, target_lens_list=targets,

@@ -37,6 +37,20 @@ def delta_rule_mixer(proj: torch.Tensor, conv_w: torch.Tensor, a_log: torch.Tens
               _hip.ptr(st.tok_pos), _hip.ptr(st.tok_state), st.seq_row0.shape[0], H, G, d, dv, stream)
     out = torch.empty((n, H * dv), dtype=proj.dtype, device=dev)
     gate = proj[:, mixer.conv_channels:mixer.conv_channels + H * dv]
-    _hip.call("swl_gated_head_rmsnorm", _hip.ptr(out), _hip.ptr(o), _hip.ptr(gate), proj.stride(0), _hip.ptr(norm_w),
-              float(eps), n, H, dv, code, stream)
+    gated_head_rmsnorm(out, o, gate, norm_w, H, dv, eps)
     return out
+
+
+def gated_head_rmsnorm(out: torch.Tensor, o: torch.Tensor, gate: torch.Tensor, norm_w: torch.Tensor, num_heads: int, vdim: int,
+                       eps: float, mult: float = 1.0):
+    """out[t, h] = mult * o / rms(o over the head) * norm_w * silu(gate): o fp32 [T, heads * vdim], gate and out rows of the compute
+    dtype (column slices are fine), norm_w fp32 with one row of vdim for all heads or one per head."""
+    _hip.require_gpu_tensor(o, "o")
+    n = o.shape[0]
+    assert o.dtype == norm_w.dtype == torch.float32 and o.is_contiguous() and o.shape[1] == num_heads * vdim
+    assert norm_w.is_contiguous() and norm_w.numel() in (vdim, num_heads * vdim)
+    for t in (gate, out):
+        assert t.shape == (n, num_heads * vdim) and t.stride(1) == 1 and t.dtype == out.dtype
+    _hip.call("swl_gated_head_rmsnorm", _hip.ptr(out), out.stride(0), _hip.ptr(o), _hip.ptr(gate), gate.stride(0),
+              _hip.ptr(norm_w), vdim if norm_w.numel() != vdim else 0, float(mult), float(eps), n, num_heads, vdim,
+              _hip.dtype_code3(out.dtype), _hip.stream())

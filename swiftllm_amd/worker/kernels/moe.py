@@ -114,6 +114,17 @@ ACT_SILU = 1        # silu(g) * u
 ACT_SILU_UP_FIRST = 2       # the same on rows [up | gate] (gated_unit only)
 
 
+def gated_rows(out: torch.Tensor, gate: torch.Tensor, up: torch.Tensor, act: int = ACT_SILU, limit: float = 0.0):
+    """out = act(gate, up) element by element; gate and up are column slices of the same rows (up after gate), out rows may be a
+    column slice too."""
+    n, ff = out.shape
+    esize = out.element_size()
+    assert gate.shape == up.shape == (n, ff) and gate.dtype == up.dtype == out.dtype and gate.stride() == up.stride()
+    assert gate.stride(1) == out.stride(1) == 1 and act in (ACT_CLAMPED, ACT_SILU)
+    _hip.call("swl_glu_rows", _hip.ptr(out), out.stride(0), _hip.ptr(gate), gate.stride(0), (up.data_ptr() - gate.data_ptr()) // esize,
+              0, n, ff, float(limit), int(act), _hip.dtype_code3(out.dtype), _hip.stream())
+
+
 def gated_unit(gu: torch.Tensor, ff: int, act: int = ACT_SILU, limit: float = 0.0, in_w: torch.Tensor = None) -> torch.Tensor:
     """[rows, gate | up] (products of a fused gate/up projection) -> [rows, ff] through the gated unit `act`. in_w (fp32 [rows]):
     a weight on the projection's input, applied to its products."""

@@ -63,6 +63,19 @@ class StateRef:
         self.tok_seq, self.seq_row0, self.seq_cnt = tok_seq, seq_row0, seq_cnt
 
 
+def token_shift_mix(h: torch.Tensor, mu: torch.Tensor, st: StateRef, tail_off: int) -> torch.Tensor:
+    """-> [mixes, T, width]: h[t] + (h[t - 1] - h[t]) * mu[s] for every row of mu (fp32 [mixes, width]); zeros stand before a
+    sequence's first token, and its last h is carried at `tail_off` inside the state slot."""
+    _hip.require_gpu_tensor(h, "h")
+    n, c = h.shape
+    assert h.stride(1) == 1 and mu.dtype == torch.float32 and mu.is_contiguous() and mu.shape[1] == c
+    out = torch.empty((mu.shape[0], n, c), dtype=h.dtype, device=h.device)
+    _hip.call("swl_token_shift_mix", _hip.ptr(out), _hip.ptr(h), h.stride(0), _hip.ptr(mu), mu.shape[0], _hip.ptr(st.pool),
+              st.pool.stride(0), int(tail_off), _hip.ptr(st.tok_pos), _hip.ptr(st.tok_start), _hip.ptr(st.tok_state),
+              _hip.ptr(st.tok_seq), n, c, _hip.dtype_code3(h.dtype), _hip.stream())
+    return out
+
+
 def causal_conv_state(h: torch.Tensor, w: torch.Tensor, st: StateRef, tail_off: int, add_input: bool) -> torch.Tensor:
     """(h +) causal convolution of h over time per channel; w fp32, tap-major [taps, channels] (the last row multiplies the
     current token); the last taps - 1 inputs of every sequence are carried at `tail_off` inside its state slot."""

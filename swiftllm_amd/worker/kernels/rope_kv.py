@@ -73,6 +73,39 @@ def qk_norm_rope_and_store_kv(rows: torch.Tensor, q_b: torch.Tensor, k_b: torch.
     return q
 
 
+def qkv_conv_rope_and_store_kv(rows: torch.Tensor, bias: torch.Tensor, conv_w: torch.Tensor, q_norm: torch.Tensor,
+                               k_norm: torch.Tensor, freq: torch.Tensor, rot, pool: torch.Tensor, pool_slice: PoolSlice,
+                               block_table: torch.Tensor, st, tail_off: int, num_q_heads: int, num_kv_heads: int, dim: int,
+                               vdim: int, k_dim: int, v_dim: int, eps: float, v_mult: float = 1.0) -> torch.Tensor:
+    """rows [q | k | v (| anything)] of one fused projection -> the queries [T, num_q_heads * k_dim]; keys and values go to the
+    pool. Per channel: + bias (fp32 [q | k | v]), causal convolution over the sequence (conv_w fp32 tap-major [taps, q | k | v],
+    carried inputs at tail_off inside the state slot); per q / k head: RMS norm with q_norm / k_norm, rotation; values times v_mult.
+    Every step optional (None). st: the step's StateRef. k_dim / v_dim: row sizes in the pool and in the result, columns beyond the
+    head zero. pool None (memory profiling): queries only."""
+    _hip.require_gpu_tensor(rows, "rows")
+    n = rows.shape[0]
+    channels = (num_q_heads + num_kv_heads) * dim + num_kv_heads * vdim
+    assert rows.dim() == 2 and rows.stride(1) == 1 and rows.shape[1] >= channels and st.tok_pos.shape[0] == n
+    for t, size in ((bias, channels), (q_norm, dim), (k_norm, dim)):
+        assert t is None or (t.dtype == torch.float32 and t.is_contiguous() and t.numel() == size)
+    assert conv_w is None or (conv_w.dtype == torch.float32 and conv_w.is_contiguous() and conv_w.shape[1] == channels)
+    rot_dims = rot.dims if freq is not None else 0
+    assert freq is None or (freq.dtype == torch.float64 and freq.numel() == rot_dims // 2)
+    kp, vp, stride = _pool_ptrs(pool, pool_slice)
+    if pool is not None:
+        assert pool.dtype == rows.dtype and block_table.is_contiguous()
+    q = torch.empty((n, num_q_heads * k_dim), dtype=rows.dtype, device=rows.device)
+    slots = st.pool if conv_w is not None else None
+    _hip.call("swl_qkv_conv_rope_store_kv", _hip.ptr(rows), rows.stride(0), _hip.ptr(q), q.stride(0), _hip.ptr(bias),
+              _hip.ptr(conv_w), conv_w.shape[0] if conv_w is not None else 0, _hip.ptr(q_norm), _hip.ptr(k_norm), _hip.ptr(freq),
+              rot_dims, 1 if rot_dims == 0 or rot.half else 0, float(rot.multiplier) if rot_dims else 1.0, float(v_mult), kp, vp,
+              _hip.ptr(block_table), block_table.shape[1] if block_table is not None else 0, stride, _hip.ptr(slots),
+              slots.stride(0) if slots is not None else 0, int(tail_off), _hip.ptr(st.tok_pos), _hip.ptr(st.tok_start),
+              _hip.ptr(st.tok_state), _hip.ptr(st.tok_seq), n, num_q_heads, num_kv_heads, dim, vdim, k_dim, v_dim, float(eps),
+              _hip.dtype_code3(rows.dtype), _hip.stream())
+    return q
+
+
 def latent_rope_and_store_kv(proj: torch.Tensor, qa: torch.Tensor, freq: torch.Tensor, c_norm: torch.Tensor,
                              pool: torch.Tensor, pool_slice: PoolSlice, block_table: torch.Tensor, tok_seq: torch.Tensor,
                              tok_pos: torch.Tensor, mixer, dkv_col: int, eps: float, k_dim: int = 0, v_dim: int = 0):

@@ -9,12 +9,12 @@ from .rms_stream import StateRef
 
 def state_space_mixer(proj: torch.Tensor, conv_w: torch.Tensor, conv_b: torch.Tensor, a_log: torch.Tensor,
                       dt_bias: torch.Tensor, d_skip: torch.Tensor, norm_w: torch.Tensor, st: StateRef, tail_off: int,
-                      state_off: int, mixer, eps: float) -> torch.Tensor:
+                      state_off: int, mixer, eps: float, out: torch.Tensor = None) -> torch.Tensor:
     """proj [T, z | x | B | C | dt] (rows of the input projection; a column slice of a wider matrix is fine) -> [T, heads * vdim]
     in proj's dtype: causal convolution with bias + SiLU on x | B | C (conv_w tap-major [taps, channels]), dt = softplus(dt +
     dt_bias), the token-by-token recurrence S <- exp(-exp(A_log) dt) S + dt B x^T, y = S^T C + D x on the fp32 state
     [heads, state, vdim] at `state_off` inside each sequence's slot, then y * silu(z) RMS-normed in mixer.norm_groups parts and
-    scaled by norm_w."""
+    scaled by norm_w. out: rows to write (a column slice is fine)."""
     _hip.require_gpu_tensor(proj, "proj")
     n = proj.shape[0]
     H, P, N, G = mixer.num_heads, mixer.value_dim, mixer.state_dim, mixer.groups
@@ -36,7 +36,9 @@ def state_space_mixer(proj: torch.Tensor, conv_w: torch.Tensor, conv_b: torch.Te
     _hip.call("swl_ssd_scan", _hip.ptr(y), _hip.ptr(xbc), _hip.ptr(dt), _hip.ptr(decay), _hip.ptr(d_skip), _hip.ptr(st.pool),
               st.pool.stride(0), int(state_off), _hip.ptr(st.seq_row0), _hip.ptr(st.seq_cnt), _hip.ptr(st.tok_pos),
               _hip.ptr(st.tok_state), st.seq_row0.shape[0], H, P, N, G, stream)
-    out = torch.empty((n, H * P), dtype=proj.dtype, device=dev)
-    _hip.call("swl_gated_group_rmsnorm", _hip.ptr(out), _hip.ptr(y), _hip.ptr(proj), proj.stride(0), _hip.ptr(norm_w),
+    if out is None:
+        out = torch.empty((n, H * P), dtype=proj.dtype, device=dev)
+    assert out.shape == (n, H * P) and out.stride(1) == 1 and out.dtype == proj.dtype
+    _hip.call("swl_gated_group_rmsnorm", _hip.ptr(out), out.stride(0), _hip.ptr(y), _hip.ptr(proj), proj.stride(0), _hip.ptr(norm_w),
               float(eps), n, H * P, mixer.norm_groups, code, stream)
     return out

@@ -178,17 +178,19 @@ MASK_CHUNK = 1      # keys [floor(p / window) * window, p]
 class AttentionSpec:
     """Shape and constants of one attention over the pool, as the kernels see it (which need not be how the design counts
     its heads: two score maps over shared values are 2 H query heads, 2 G key heads and G value heads).
-    num_v_heads: value heads in a page; key head g reads value head g % num_v_heads. window: sliding window or chunk size
+    num_v_heads: value heads in a page; key head g reads value head g % num_v_heads. slopes: fp32 [num_q_heads], slope times the
+    distance query - key is taken off the score, or None. out_dim: value columns that count (the pages' rows may be wider). window: sliding window or chunk size
     (mask_kind), 0 for every earlier key. sink: fp32 [num_q_heads] logits that join the denominators, or None."""
     __slots__ = ("num_q_heads", "num_kv_heads", "num_v_heads", "head_dim", "value_dim", "window", "mask_kind", "scale",
-                 "softcap", "sink", "out_f32")
+                 "softcap", "sink", "out_f32", "slopes", "out_dim")
 
     def __init__(self, num_q_heads, num_kv_heads, head_dim, value_dim, scale, window=0, mask_kind=MASK_WINDOW,
-                 num_v_heads=None, softcap=0.0, sink=None, out_f32=False):
+                 num_v_heads=None, softcap=0.0, sink=None, out_f32=False, slopes=None, out_dim=None):
         self.num_q_heads, self.num_kv_heads, self.head_dim, self.value_dim = num_q_heads, num_kv_heads, head_dim, value_dim
         self.num_v_heads = num_kv_heads if num_v_heads is None else num_v_heads
         self.window, self.mask_kind, self.scale, self.softcap, self.sink, self.out_f32 = \
             window, mask_kind, scale, softcap, sink, out_f32
+        self.slopes, self.out_dim = slopes, value_dim if out_dim is None else out_dim
 
 
 def masked_tiles_supported(spec: AttentionSpec, dtype: torch.dtype) -> bool:
@@ -234,8 +236,9 @@ def choose_heads_per_group(spec: AttentionSpec) -> int:
 
 def masked_attention(q: torch.Tensor, pool: torch.Tensor, pool_slice: PoolSlice, block_table: torch.Tensor,
                      tok_seq: torch.Tensor, tok_pos: torch.Tensor, spec: AttentionSpec, tiles=None,
-                     max_positions: int = 1 << 20) -> torch.Tensor:
-    """-> [T, num_q_heads * value_dim] (fp32 when spec.out_f32, else q's dtype). q: rows whose first num_q_heads * head_dim
+                     max_positions: int = 1 << 20, out: torch.Tensor = None, gate: torch.Tensor = None) -> torch.Tensor:
+    """-> [T, num_q_heads * out_dim] (fp32 when spec.out_f32, else q's dtype), written to `out` when given (a column slice of wider
+    rows is fine), times sigmoid(gate) element by element when `gate` (likewise) is. q: rows whose first num_q_heads * head_dim
     columns are the queries (a column slice of a wider matrix is fine); keys and values come from the pool, which already
     holds this step's tokens."""
     _hip.require_gpu_tensor(q, "q")
@@ -243,13 +246,18 @@ def masked_attention(q: torch.Tensor, pool: torch.Tensor, pool_slice: PoolSlice,
     assert pool.is_contiguous() and pool.dtype == q.dtype and tok_pos.dtype == torch.int32 and tok_seq.dtype == torch.int32
     sink = spec.sink
     assert sink is None or (sink.dtype == torch.float32 and sink.is_contiguous() and sink.numel() == spec.num_q_heads)
-    n = q.shape[0]
-    out = torch.empty((n, spec.num_q_heads * spec.value_dim), dtype=torch.float32 if spec.out_f32 else q.dtype,
-                      device=q.device)
+    n, cols = q.shape[0], spec.num_q_heads * spec.out_dim
+    assert spec.slopes is None or (spec.slopes.dtype == torch.float32 and spec.slopes.numel() == spec.num_q_heads)
+    if out is None:
+        out = torch.empty((n, cols), dtype=torch.float32 if spec.out_f32 else q.dtype, device=q.device)
+    assert out.shape == (n, cols) and out.stride(1) == 1 and (out.dtype == torch.float32 if spec.out_f32 else out.dtype == q.dtype)
+    assert gate is None or (gate.shape == (n, cols) and gate.stride(1) == 1 and gate.dtype == q.dtype)
+    gate_stride = gate.stride(0) if gate is not None else 0
     esize = pool.element_size()
     kp = pool.data_ptr() + pool_slice.k_offset * esize
     vp = pool.data_ptr() + pool_slice.v_offset * esize
     wide_ok = q.stride(0) % 4 == 0 and q.data_ptr() % 8 == 0 and kp % 8 == 0 and vp % 8 == 0 and pool.shape[1] % 4 == 0
+    wide_ok = wide_ok and out.data_ptr() % (16 if spec.out_f32 else 8) == 0 and out.stride(0) % 4 == 0
     if tiles is not None and wide_ok and masked_tiles_supported(spec, q.dtype):
         row0, cnt = tiles
         if spec.num_kv_heads == 1 and row0.shape[0] == n and spec.num_q_heads >= HEAD_ROWS_MIN_HEADS:
@@ -267,10 +275,12 @@ def masked_attention(q: torch.Tensor, pool: torch.Tensor, pool_slice: PoolSlice,
                   _hip.ptr(tok_pos), _hip.ptr(row0), _hip.ptr(cnt), 0, 0, 0, row0.shape[0], spec.num_q_heads,
                   spec.num_kv_heads, spec.head_dim, spec.value_dim, q.stride(0), spec.window, float(spec.scale),
                   float(spec.softcap), block_table.shape[1], pool.shape[1], splits, _hip.ptr(scratch), n, spec.mask_kind,
-                  _hip.ptr(sink), spec.num_v_heads, 1 if spec.out_f32 else 0, hpg, _hip.dtype_code(q.dtype), _hip.stream())
+                  _hip.ptr(sink), spec.num_v_heads, 1 if spec.out_f32 else 0, hpg, _hip.ptr(spec.slopes), spec.out_dim,
+                  out.stride(0), _hip.ptr(gate), gate_stride, _hip.dtype_code(q.dtype), _hip.stream())
         return out
     _hip.call("swl_masked_attn", _hip.ptr(out), _hip.ptr(q), kp, vp, _hip.ptr(block_table), _hip.ptr(tok_seq),
               _hip.ptr(tok_pos), 0, 0, 0, n, spec.num_q_heads, spec.num_kv_heads, spec.head_dim, spec.value_dim, q.stride(0),
               spec.window, float(spec.scale), float(spec.softcap), block_table.shape[1], pool.shape[1], spec.mask_kind,
-              _hip.ptr(sink), spec.num_v_heads, 1 if spec.out_f32 else 0, _hip.dtype_code3(q.dtype), _hip.stream())
+              _hip.ptr(sink), spec.num_v_heads, 1 if spec.out_f32 else 0, _hip.ptr(spec.slopes), spec.out_dim, out.stride(0),
+              _hip.ptr(gate), gate_stride, _hip.dtype_code3(q.dtype), _hip.stream())
     return out
