@@ -96,9 +96,9 @@ def parse_args():
     ap.add_argument("--no-reference", action="store_true", help="skip the reference-Triton child run")
     ap.add_argument("--compare-designs", action="store_true",
                     help="instead of the headline workload: prefill and decode throughput of the other designs (Kekapel, "
-                         "Lorulix, Rosilix, Ratilorn, Rokevik) beside LLaMA at equal layer sizes (random weights), one "
+                         "Lorulix, Rosilix, Ratilorn, Rokevik, Vafozen) beside LLaMA at equal layer sizes (random weights), one "
                          "JSON line with all")
-    ap.add_argument("--compare", default="llama,kekapel,lorulix,rosilix,ratilorn,rokevik",
+    ap.add_argument("--compare", default="llama,kekapel,lorulix,rosilix,ratilorn,rokevik,vafozen",
                     help="designs that --compare-designs runs (comma list)")
     ap.add_argument("--compare-kv-rank", type=int, default=512,
                     help="latent size of Rosilix's and Rokevik's latent attention layers in --compare-designs")
@@ -192,7 +192,20 @@ def _compare_configs(sz, positions, kv_rank=512):
     klayers = [dict(type=kinds[i % 4][0], mixer=dict(kinds[i % 4][1]), mlp=kmoe) for i in range(sz["layers"])]
     rokevik = dict(architecture="Rokevik", layers=klayers, max_positions=positions, norm=dict(eps=1e-6, groups=2), streams=2,
                    logit_softcap=30.0, vocab=sz["vocab"], width=sz["width"])
-    return llama, kekapel, lorulix, rosilix, ratilorn, rokevik
+    # Vafozen at the same sizes: chunked attention beside gated linear attention / convolved rotary attention beside time mixing /
+    # a state-space recurrence of Ratilorn's sizes, in turn (recurrences: heads of dim x dim states); dense feed-forwards
+    chunked = dict(dim=sz["dim"], vdim=sz["dim"], heads=sz["heads"], kv_heads=sz["kv_heads"], scale=sz["dim"] ** -0.5,
+                   mask=dict(size=1024))
+    convolved = dict(dim=sz["dim"], vdim=sz["dim"], heads=sz["heads"], kv_heads=sz["kv_heads"], scale=sz["dim"] ** -0.5, conv=4,
+                     softcap=30.0, rot=dict(base=10000.0, dims=sz["dim"]))
+    vkinds = (("parallel", dict(left=chunked, right=dict(heads=sz["heads"], dim=sz["dim"], vdim=sz["dim"], tau=16.0),
+                                left_scale=0.8, right_scale=1.1)),
+              ("parallel_2", dict(left=convolved, right=dict(heads=sz["heads"], dim=sz["dim"]), left_scale=0.8, right_scale=1.1)),
+              ("mamba2", dict(par["right"])))
+    vlayers = [dict(type=vkinds[i % 3][0], mixer=vkinds[i % 3][1], mlp=dict(kind="dense", ff=sz["ff"])) for i in range(sz["layers"])]
+    vafozen = dict(architecture="Vafozen", embedding=dict(scale=1.0), layers=vlayers, max_positions=positions, norm=dict(eps=1e-6),
+                   vocab=sz["vocab"], width=sz["width"])
+    return llama, kekapel, lorulix, rosilix, ratilorn, rokevik, vafozen
 
 
 def _compare_one(cfg, dtype, prompt_len, prompt_batch, decode_batch, decode_ctx, steps, warmup):
@@ -258,12 +271,12 @@ def run_compare_designs(args):
     each of the three: Kekapel is its closest, an all-attention design on the same worker and attention kernels, and Ratilorn
     over Lorulix — its closest: attention beside a recurrence with state slots, experts with a shared one — Kekapel and
     LLaMA; Rokevik over Rosilix — its closest mixers: latent attention and rotary heads — Ratilorn — its closest feed-forwards and
-    state slots — Kekapel and LLaMA)."""
+    state slots — Kekapel and LLaMA; Vafozen over Ratilorn — its closest: attention beside a recurrence — Kekapel and LLaMA)."""
     results = {}
     for name in [s for s in args.compare_sizes.split(",") if s]:
         sz = COMPARE_SIZES[name]
         prompt_len, prompt_batch, decode_batch, decode_ctx = 2048, 4, 32, 1024
-        configs = dict(zip(("llama", "kekapel", "lorulix", "rosilix", "ratilorn", "rokevik"),
+        configs = dict(zip(("llama", "kekapel", "lorulix", "rosilix", "ratilorn", "rokevik", "vafozen"),
                            _compare_configs(sz, prompt_len + 256, args.compare_kv_rank)))
         rec = {"sizes": sz, "prompt": [prompt_batch, prompt_len], "decode": [decode_batch, decode_ctx]}
         for label in [d for d in args.compare.split(",") if d]:
@@ -276,7 +289,8 @@ def run_compare_designs(args):
                           ("ratilorn", "lorulix", "ratilorn_vs_lorulix_"), ("ratilorn", "kekapel", "ratilorn_vs_kekapel_"),
                           ("ratilorn", "llama", "ratilorn_vs_llama_"), ("rokevik", "rosilix", "rokevik_vs_rosilix_"),
                           ("rokevik", "ratilorn", "rokevik_vs_ratilorn_"), ("rokevik", "kekapel", "rokevik_vs_kekapel_"),
-                          ("rokevik", "llama", "rokevik_vs_llama_")):
+                          ("rokevik", "llama", "rokevik_vs_llama_"), ("vafozen", "ratilorn", "vafozen_vs_ratilorn_"),
+                          ("vafozen", "kekapel", "vafozen_vs_kekapel_"), ("vafozen", "llama", "vafozen_vs_llama_")):
             if a in rec and b in rec:
                 rec[key + "prefill_ratio"] = rec[a]["prefill_tokens_per_s"] / rec[b]["prefill_tokens_per_s"]
                 rec[key + "decode_ratio"] = rec[a]["decode_tokens_per_s"] / rec[b]["decode_tokens_per_s"]
