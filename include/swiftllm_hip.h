@@ -262,6 +262,11 @@ int swl_gemm_pack_weight(void *dst, const void *src, int32_t N, int32_t K, int32
 int swl_gemm_skinny_packed(void *out, const void *x, const void *w_packed, void *workspace, size_t workspace_bytes,
                            int32_t M, int32_t N, int32_t K, int64_t x_row_stride, int64_t out_row_stride,
                            int32_t k_splits, int32_t dtype, swl_stream_t stream);
+/* swl_gemm_skinny_packed for several inputs at once: columns g * N / groups .. of the result are the product of the rows at
+ * x + g * x_group_stride with the weight's rows of those numbers; N / groups a multiple of 128. */
+int swl_gemm_skinny_packed_grouped(void *out, const void *x, int64_t x_group_stride, int32_t groups, const void *w_packed,
+                                   void *workspace, size_t workspace_bytes, int32_t M, int32_t N, int32_t K, int64_t x_row_stride,
+                                   int64_t out_row_stride, int32_t dtype, swl_stream_t stream);
 int swl_gemm_skinny_packed_partial(float *slabs, size_t slabs_bytes, const void *x, const void *w_packed, int32_t M,
                                    int32_t N, int32_t K, int64_t x_row_stride, int32_t k_splits, int32_t dtype,
                                    swl_stream_t stream);
@@ -837,13 +842,14 @@ int swl_low_rank_decay(float *out, const void *x, int64_t x_stride, const void *
 
 /* ---- fp32 residual of several streams, hyper-connections (csrc/hyper_stream.hip) ------------------------------------------------
  * x [rows, streams, width] fp32. swl_embed_streams: every stream = embed[token]. swl_hyper_step: with y (+ y2, + y_bias[width])
- * the previous sublayer's result (the fp32 sum of y_parts rows y[t * y_parts + j]), X_t <- sum_s mix[s][t] X_s + outw[t] y (all from the old streams); then, with h given,
+ * the previous sublayer's result (the fp32 sum of y_parts rows y[t * y_parts + j], or — y NULL, slabs given — of the y_parts fp32
+ * slabs [rows, width] that lie slab_stride elements apart: a product's K shares), X_t <- sum_s mix[s][t] X_s + outw[t] y (all from the old streams); then, with h given,
  * u = sum_s inw[s] X_s (inw NULL: plain sum) and h = u / rms(u in `groups` equal parts; eps) * norm_w. y NULL: norm only, of
  * rows row_idx when given; h NULL: update only. At most 16 streams. dtype (y, y2, h) may be SWL_F32. */
 int swl_embed_streams(float *x, const void *embed, const int32_t *tokens, int64_t num_tokens, int32_t width, int32_t streams,
                       int32_t dtype, swl_stream_t stream);
-int swl_hyper_step(float *x, const void *y, int32_t y_parts, const void *y2, const float *y_bias, const float *mix,
-                   const float *outw, const float *inw, const float *norm_w, void *h, const int32_t *row_idx, int64_t num_rows,
+int swl_hyper_step(float *x, const void *y, int32_t y_parts, const float *slabs, int64_t slab_stride, const void *y2,
+                   const float *y_bias, const float *mix, const float *outw, const float *inw, const float *norm_w, void *h, const int32_t *row_idx, int64_t num_rows,
                    int32_t width, int32_t streams, int32_t groups, float eps, int32_t dtype, swl_stream_t stream);
 
 /* ---- minGRU (csrc/min_gru.hip) -----------------------------------------------------------------------------------------------------

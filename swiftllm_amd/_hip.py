@@ -62,6 +62,7 @@ SIGNATURES = {
     "swl_gemm_skinny": [_P, _P, _P, _P, ctypes.c_size_t, _I32, _I32, _I32, _I64, _I64, _I32, _I32, _P],
     "swl_gemm_pack_weight": [_P, _P, _I32, _I32, _I32, _P],
     "swl_gemm_skinny_packed": [_P, _P, _P, _P, ctypes.c_size_t, _I32, _I32, _I32, _I64, _I64, _I32, _I32, _P],
+    "swl_gemm_skinny_packed_grouped": [_P, _P, _I64, _I32, _P, _P, ctypes.c_size_t, _I32, _I32, _I32, _I64, _I64, _I32, _P],
     "swl_gemm_packed_mid_partial": [_P, ctypes.c_size_t, _P, _P, _I32, _I32, _I32, _I64, _I32, _I32, _P],
     "swl_gemm_packed_mid_silu_gate": [_P, _P, _P, _I32, _I32, _I32, _I64, _I64, _I32, _P],
     "swl_gemm_packed_mid": [_P, _P, _P, _P, ctypes.c_size_t, _I32, _I32, _I32, _I64, _I64, _I32, _I32, _P],
@@ -146,7 +147,7 @@ SIGNATURES = {
     "swl_qk_norm_rope_store_kv": [_P, _P, _P, _P, _P, _P, _P, _P, _P, _P, _P, _P, _P, _I64, _I32, _I32, _I32, _I32, _I32, _I32,
                                   _I32, _F64, _I64, _I64, _I32, _I32, _I32, _I32, _I64, _F32, _I32, _P],
     "swl_embed_streams": [_P, _P, _P, _I64, _I32, _I32, _I32, _P],
-    "swl_hyper_step": [_P, _P, _I32, _P, _P, _P, _P, _P, _P, _P, _P, _I64, _I32, _I32, _I32, _F32, _I32, _P],
+    "swl_hyper_step": [_P, _P, _I32, _P, _I64, _P, _P, _P, _P, _P, _P, _P, _P, _I64, _I32, _I32, _I32, _F32, _I32, _P],
     "swl_min_gru_chunks": [_P, _P, _I64, _P, _P, _P, _P, _I32, _I32, _I32, _P],
     "swl_min_gru_carry": [_P, _P, _I64, _I64, _P, _P, _P, _P, _P, _I32, _I32, _I32, _P],
     "swl_min_gru_apply": [_P, _P, _I64, _P, _P, _P, _P, _I64, _I64, _P, _P, _P, _P, _I32, _I32, _I32, _P],

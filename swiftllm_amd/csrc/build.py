@@ -58,7 +58,7 @@ MODEL_SOURCES = {
     "Rosilix": _SHARED + ["layernorm.hip", "window_attn.hip", "window_attn_mfma.hip", "moe.hip", "rms_stream.hip",
                           "rope_kv.hip"],
     "Ratilorn": _SHARED + ["layernorm.hip", "qknorm_kv.hip", "window_attn.hip", "window_attn_mfma.hip", "moe.hip",
-                           "rms_stream.hip", "sigmoid_attn.hip", "ssd.hip"],
+                           "rms_stream.hip", "sigmoid_attn.hip", "ssd.hip", "linear_scan.hip", "delta_rule.hip"],
     "Rokevik": _SHARED + ["window_attn.hip", "window_attn_mfma.hip", "moe.hip", "rope_kv.hip", "hyper_stream.hip", "min_gru.hip"],
     "Vafozen": _SHARED + ["layernorm.hip", "window_attn.hip", "window_attn_mfma.hip", "moe.hip", "rms_stream.hip", "rope_kv.hip",
                           "hyper_stream.hip", "delta_rule.hip", "ssd.hip", "linear_scan.hip", "low_rank_decay.hip"],

@@ -71,6 +71,10 @@ struct GemmExtra {
     // ssq_out[ksplit][M] (the row_ssq the slab-fed attention prologue takes)
     const void *norm_w;
     float *ssq_out;
+    // grouped inputs (direct and partial modes): > 0 = columns per group (a multiple of a workgroup's); the columns of group g
+    // multiply the rows at x + g * x_group_stride
+    int x_group_cols;
+    int64_t x_group_stride;
 };
 
 // acc[r] = out^T[n = n0 + (r&3) + 8*(r>>2) + 4*hf][m = l32] -> the three output modes.
@@ -267,6 +271,8 @@ __global__ __launch_bounds__(NWV * 64, NWV == 2 ? 1 : 2) void gemm_skinny_ring_k
     const bool is_gate = MODE == kGemmSiluGate && wave >= HWV;
     const int col0 = MODE == kGemmSiluGate ? (blockIdx.x * HWV + (wave % HWV)) * 32
                                            : (blockIdx.x * NWV + wave) * 32;
+    if (PACKED && !NF && MODE != kGemmSiluGate && fuse.x_group_cols > 0)
+        x += (static_cast<int>(blockIdx.x) * NWV * 32 / fuse.x_group_cols) * fuse.x_group_stride;
     const bool tile_ok = col0 < N; // barriers below: a wave without a tile still stages x and syncs
     const int n0 = tile_ok ? col0 + (is_gate ? N : 0) : 0;
     const int ksplit = blockIdx.y;
@@ -744,7 +750,7 @@ static void launch_packed(dim3 grid, hipStream_t stream, void *out, const T *x, 
 
 template <typename T>
 static int run_gemm_packed(T *out, const T *x, const T *wp, float *ws, size_t ws_bytes, int M, int N, int K, int64_t xs,
-                           int64_t os, int ks, hipStream_t stream, bool reduce) {
+                           int64_t os, int ks, hipStream_t stream, bool reduce, int group_cols = 0, int64_t group_stride = 0) {
     bool uneven = false;
     if (ks <= 0) ks = choose_k_splits_packed(N, K, &uneven);
     else uneven = K % (kKT * ks) != 0;
@@ -752,13 +758,18 @@ static int run_gemm_packed(T *out, const T *x, const T *wp, float *ws, size_t ws
     const dim3 grid((N / 32 + kGemmWaves - 1) / kGemmWaves, ks);
     const int kc = uneven ? (K / kKT / ks) * kKT : K / ks;  // (uneven: the shorter chunk — selects the ring depth)
     if (ks == 1 && reduce) {
-        launch_packed<T, kGemmDirect>(grid, stream, out, x, wp, M, N, K, kc, xs, os);
+        GemmExtra fuse{};
+        fuse.x_group_cols = group_cols;
+        fuse.x_group_stride = group_stride;
+        launch_packed<T, kGemmDirect>(grid, stream, out, x, wp, M, N, K, kc, xs, os, fuse);
         return check_launch();
     }
     if (!ws || ws_bytes < static_cast<size_t>(ks) * M * N * sizeof(float)) return SWL_ERR_BAD_ARG;
     GemmExtra fuse{};
     fuse.k_tiles_total = uneven ? K / kKT : 0;
-    if (!uneven && prefer_three_waves(N, ks)) launch_packed_partial3<T>(stream, ws, x, wp, M, N, K, kc, ks, xs);
+    fuse.x_group_cols = group_cols;
+    fuse.x_group_stride = group_stride;
+    if (!uneven && group_cols == 0 && prefer_three_waves(N, ks)) launch_packed_partial3<T>(stream, ws, x, wp, M, N, K, kc, ks, xs);
     else launch_packed<T, kGemmPartial>(grid, stream, ws, x, wp, M, N, K, kc, xs, static_cast<int64_t>(N), fuse);
     if (!reduce) return check_launch();
     const int64_t items = static_cast<int64_t>(M) * (N / 4);
@@ -804,6 +815,25 @@ extern "C" int swl_gemm_skinny_packed(void *out, const void *x, const void *w_pa
                                        static_cast<const T *>(w_packed), static_cast<float *>(workspace),
                                        workspace_bytes, M, N, K, x_row_stride, out_row_stride, k_splits,
                                        static_cast<hipStream_t>(stream), true);
+    });
+}
+
+extern "C" int swl_gemm_skinny_packed_grouped(void *out, const void *x, int64_t x_group_stride, int32_t groups, const void *w_packed,
+                                              void *workspace, size_t workspace_bytes, int32_t M, int32_t N, int32_t K,
+                                              int64_t x_row_stride, int64_t out_row_stride, int32_t dtype, swl_stream_t stream) {
+    if (M < 0 || N <= 0 || K <= 0 || groups <= 0 || N % groups) return SWL_ERR_BAD_ARG;
+    if (M == 0) return SWL_OK;
+    if (!out || !x || !w_packed) return SWL_ERR_BAD_ARG;
+    if (M > 32 || (K & (swl::kKT - 1)) || (N / groups) % (swl::kGemmWaves * 32)) return SWL_ERR_UNSUPPORTED;
+    if (x_row_stride < K || out_row_stride < N || (x_row_stride & 7) || (x_group_stride & 7) || (out_row_stride & 3))
+        return SWL_ERR_BAD_ARG;
+    if (!swl::aligned16(x) || !swl::aligned16(w_packed) || (reinterpret_cast<uintptr_t>(out) & 7u) ||
+        (workspace && !swl::aligned16(workspace)))
+        return SWL_ERR_BAD_ARG;
+    SWL_DISPATCH_DTYPE(dtype, T, {
+        return swl::run_gemm_packed<T>(static_cast<T *>(out), static_cast<const T *>(x), static_cast<const T *>(w_packed),
+                                       static_cast<float *>(workspace), workspace_bytes, M, N, K, x_row_stride, out_row_stride, 0,
+                                       static_cast<hipStream_t>(stream), true, N / groups, x_group_stride);
     });
 }
 

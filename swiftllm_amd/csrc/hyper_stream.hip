@@ -2,7 +2,8 @@
 //
 //   swl_embed_streams: x[t][s] = embed[token[t]] for every stream s.
 //   swl_hyper_step:    the step between two sublayers in one launch, one workgroup per token. With the previous sublayer's result
-//                      y (the sum of y_parts rows per token: the results of a token's experts; + y2: a second addend, + y_bias: a
+//                      y (the sum of y_parts rows per token: the results of a token's experts, or of fp32 slabs: the K shares of
+//                      the product that makes it; + y2: a second addend, + y_bias: a
 //                      bias of its output projection)
 //       X_t <- sum_s mix[s][t] X_s + out[t] * y        all streams at once from the old ones
 //       u    = sum_s in[s] X_s                         what the next sublayer reads
@@ -57,7 +58,8 @@ __device__ __forceinline__ void hs_store(T *p, const float *src) {
 // S: streams held in registers (S == streams when EXACT, else S >= streams). V: columns per access (4 when width % 4 == 0).
 template <typename T, int S, int V, bool EXACT>
 __global__ __launch_bounds__(kHsThreads) void hyper_step_kernel(
-    float *x, const T *y, int y_parts, const T *y2, const float *y_bias, const float *__restrict__ mix, const float *__restrict__ outw,
+    float *x, const T *y, int y_parts, const float *slabs, int64_t slab_stride, const T *y2, const float *y_bias,
+    const float *__restrict__ mix, const float *__restrict__ outw,
     const float *__restrict__ inw, const float *__restrict__ norm_w, T *h, const int32_t *row_idx, int width, int streams,
     int groups, float eps) {
     extern __shared__ float lds[];
@@ -87,14 +89,31 @@ __global__ __launch_bounds__(kHsThreads) void hyper_step_kernel(
         float u[V];
 #pragma unroll
         for (int j = 0; j < V; ++j) u[j] = 0.f;
-        if (y) {
+        if (y || slabs) {
             float yv[V];
-            hs_load<T, V>(yv, y + t * y_parts * width + c);
-            for (int k = 1; k < y_parts; ++k) {
-                float b[V];
-                hs_load<T, V>(b, y + (t * y_parts + k) * width + c);
+            if (slabs) {        // (four at a time: requested before the first sum)
+                const float *p = slabs + t * width + c;
+                hs_load<float, V>(yv, p);
+                for (int k = 1; k < y_parts; k += 4) {
+                    float b[4][V];
 #pragma unroll
-                for (int j = 0; j < V; ++j) yv[j] += b[j];
+                    for (int u = 0; u < 4; ++u) hs_load<float, V>(b[u], p + min(k + u, y_parts - 1) * slab_stride);
+#pragma unroll
+                    for (int u = 0; u < 4; ++u) {
+                        if (k + u < y_parts) {
+#pragma unroll
+                            for (int j = 0; j < V; ++j) yv[j] += b[u][j];
+                        }
+                    }
+                }
+            } else {
+                hs_load<T, V>(yv, y + t * y_parts * width + c);
+                for (int k = 1; k < y_parts; ++k) {
+                    float b[V];
+                    hs_load<T, V>(b, y + (t * y_parts + k) * width + c);
+#pragma unroll
+                    for (int j = 0; j < V; ++j) yv[j] += b[j];
+                }
             }
             if (y2) {
                 float b[V];
@@ -195,11 +214,11 @@ inline size_t hs_lds_bytes(int width, int groups) {
 }
 
 template <typename T, int V>
-void launch_hs(dim3 grid, size_t lds, hipStream_t s, float *x, const T *y, int yp, const T *y2, const float *yb, const float *mix,
+void launch_hs(dim3 grid, size_t lds, hipStream_t s, float *x, const T *y, int yp, const float *sl, int64_t ss, const T *y2, const float *yb, const float *mix,
                const float *ow, const float *iw, const float *nw, T *h, const int32_t *ri, int width, int streams, int groups,
                float eps) {
 #define SWL_HS(S, X)                                                                                                          \
-    hipLaunchKernelGGL((hyper_step_kernel<T, S, V, X>), grid, dim3(kHsThreads), lds, s, x, y, yp, y2, yb, mix, ow, iw, nw, h, ri, \
+    hipLaunchKernelGGL((hyper_step_kernel<T, S, V, X>), grid, dim3(kHsThreads), lds, s, x, y, yp, sl, ss, y2, yb, mix, ow, iw, nw, h, ri, \
                        width, streams, groups, eps)
     switch (streams) {
     case 1: SWL_HS(1, true); break;
@@ -229,27 +248,30 @@ extern "C" int swl_embed_streams(float *x, const void *embed, const int32_t *tok
     return swl::check_launch();
 }
 
-extern "C" int swl_hyper_step(float *x, const void *y, int32_t y_parts, const void *y2, const float *y_bias, const float *mix,
-                              const float *outw, const float *inw, const float *norm_w, void *h, const int32_t *row_idx,
+extern "C" int swl_hyper_step(float *x, const void *y, int32_t y_parts, const float *slabs, int64_t slab_stride, const void *y2,
+                              const float *y_bias, const float *mix, const float *outw, const float *inw, const float *norm_w, void *h, const int32_t *row_idx,
                               int64_t num_rows, int32_t width, int32_t streams, int32_t groups, float eps, int32_t dtype,
                               swl_stream_t stream) {
-    if (y && y_parts < 1) return SWL_ERR_BAD_ARG;
+    const bool has_y = y || slabs;
+    if ((y && slabs) || (has_y && y_parts < 1)) return SWL_ERR_BAD_ARG;
     if (num_rows < 0 || width <= 0 || streams <= 0 || groups <= 0 || width % groups) return SWL_ERR_BAD_ARG;
     if (num_rows == 0) return SWL_OK;
-    if (!x || (y && (!mix || !outw)) || (!y && (y2 || y_bias)) || (h && !norm_w) || (row_idx && y)) return SWL_ERR_BAD_ARG;
-    if (!y && !h) return SWL_OK;
+    if (!x || (has_y && (!mix || !outw)) || (!has_y && (y2 || y_bias)) || (h && !norm_w) || (row_idx && has_y))
+        return SWL_ERR_BAD_ARG;
+    if (!has_y && !h) return SWL_OK;
     const size_t lds = swl::hs_lds_bytes(width, groups);
     if (num_rows > 0x7fffffffLL || streams > swl::kHsMaxStreams || lds > 64 * 1024) return SWL_ERR_UNSUPPORTED;
-    const bool wide = width % 4 == 0 && swl::aligned16(x) && swl::aligned16(y) && swl::aligned16(y2) && swl::aligned16(y_bias) &&
+    const bool wide = width % 4 == 0 && swl::aligned16(x) && swl::aligned16(y) && swl::aligned16(slabs) &&
+                      slab_stride % 4 == 0 && swl::aligned16(y2) && swl::aligned16(y_bias) &&
                       swl::aligned16(norm_w) && swl::aligned16(h);
     const dim3 grid(static_cast<unsigned>(num_rows));
     hipStream_t s = static_cast<hipStream_t>(stream);
     SWL_DISPATCH_DTYPE3(dtype, T, {
         if (wide)
-            swl::launch_hs<T, 4>(grid, lds, s, x, static_cast<const T *>(y), y_parts, static_cast<const T *>(y2), y_bias, mix, outw, inw,
+            swl::launch_hs<T, 4>(grid, lds, s, x, static_cast<const T *>(y), y_parts, slabs, slab_stride, static_cast<const T *>(y2), y_bias, mix, outw, inw,
                                  norm_w, static_cast<T *>(h), row_idx, width, streams, groups, eps);
         else
-            swl::launch_hs<T, 1>(grid, lds, s, x, static_cast<const T *>(y), y_parts, static_cast<const T *>(y2), y_bias, mix, outw, inw,
+            swl::launch_hs<T, 1>(grid, lds, s, x, static_cast<const T *>(y), y_parts, slabs, slab_stride, static_cast<const T *>(y2), y_bias, mix, outw, inw,
                                  norm_w, static_cast<T *>(h), row_idx, width, streams, groups, eps);
     });
     return swl::check_launch();

@@ -121,14 +121,17 @@ __device__ __forceinline__ float4_t mfma_f32_16x16x4(float a, float b, float4_t 
     return __builtin_amdgcn_mfma_f32_16x16x4f32(a, b, c, 0, 0, 0);
 }
 
+// What a wave needs of one tile. Loaded without predicates (addresses are clamped, what does not count is masked at its use): a
+// predicated load would be waited for on the spot, and the point is to have a tile's loads in flight while others are computed.
 template <typename T, int TW>
 struct LsOperands {
     float4_t q[TW], k[TW], a[TW];
-    float m, v[4];
+    float m;
+    T v[4];
 };
 
-// TW: 16-row state tiles per wave
-template <typename T, int TW>
+// TW: 16-row state tiles per wave; AHEAD: tiles requested ahead of the one being computed
+template <typename T, int TW, int AHEAD>
 __global__ __launch_bounds__(kLsThreads) void linear_scan_kernel(
     float *o, int64_t o_stride, const float *qd, const float *kd, const float *total, const float *intra, const T *v,
     int64_t v_stride, const float *dskip, float *state, int64_t slot_stride, int64_t s_off, const int32_t *seq_row0,
@@ -155,62 +158,56 @@ __global__ __launch_bounds__(kLsThreads) void linear_scan_kernel(
     }
     const float dh = dskip ? dskip[h] : 0.f;
     const int nt = (cnt + kLsTile - 1) / kLsTile;
+    const T *vcol = v + static_cast<int64_t>(row0) * v_stride + static_cast<int64_t>(h) * dv + (okc ? col : dv - 1);
     auto load = [&](int i, LsOperands<T, TW> &f) {
+        i = min(i, nt - 1);
         const int64_t at = static_cast<int64_t>(tile0 + i) * H + h;
 #pragma unroll
         for (int j = 0; j < TW; ++j) {
-            const int tl = wave * TW + j;
-            if (tl < ntiles) {
-                f.q[j] = *reinterpret_cast<const float4_t *>(qd + (at * kLsTile + li) * dp + 16 * tl + 4 * lq);
-                f.k[j] = *reinterpret_cast<const float4_t *>(kd + (at * dp + 16 * tl + li) * kLsTile + 4 * lq);
-                f.a[j] = *reinterpret_cast<const float4_t *>(total + at * dp + 16 * tl + 4 * lq);
-            }
+            const int tl = min(wave * TW + j, ntiles - 1);
+            f.q[j] = *reinterpret_cast<const float4_t *>(qd + (at * kLsTile + li) * dp + 16 * tl + 4 * lq);
+            f.k[j] = *reinterpret_cast<const float4_t *>(kd + (at * dp + 16 * tl + li) * kLsTile + 4 * lq);
+            f.a[j] = *reinterpret_cast<const float4_t *>(total + at * dp + 16 * tl + 4 * lq);
         }
         f.m = intra[at * 256 + li * kLsTile + 4 * lq + wave];
 #pragma unroll
-        for (int r = 0; r < 4; ++r) {
-            const int t = i * kLsTile + 4 * lq + r;
-            f.v[r] = (t < cnt && okc) ? to_f(v[(row0 + t) * v_stride + static_cast<int64_t>(h) * dv + col]) : 0.f;
-        }
+        for (int r = 0; r < 4; ++r) f.v[r] = vcol[static_cast<int64_t>(min(i * kLsTile + 4 * lq + r, cnt - 1)) * v_stride];
     };
-    LsOperands<T, TW> cur, nxt;
-    load(0, cur);
-    for (int i = 0; i < nt; ++i) {
-        if (i + 1 < nt) load(i + 1, nxt);
+    auto compute = [&](int i, const LsOperands<T, TW> &f) {
+        float vv[4];
+#pragma unroll
+        for (int r = 0; r < 4; ++r) vv[r] = (i * kLsTile + 4 * lq + r < cnt && okc) ? to_f(f.v[r]) : 0.f;
         // this wave's share of the outputs: its state rows, and the in-tile keys 4 lq + wave
         float4_t part[TW + 1];
-        part[TW] = mfma_f32_16x16x4(cur.m, wave == 0 ? cur.v[0] : wave == 1 ? cur.v[1] : wave == 2 ? cur.v[2] : cur.v[3],
+        part[TW] = mfma_f32_16x16x4(f.m, wave == 0 ? vv[0] : wave == 1 ? vv[1] : wave == 2 ? vv[2] : vv[3],
                                     float4_t{0.f, 0.f, 0.f, 0.f});
 #pragma unroll
-        for (int j = 0; j < TW; ++j) {
-            part[j] = float4_t{0.f, 0.f, 0.f, 0.f};
-            if (wave * TW + j < ntiles) {
+        for (int j = 0; j < TW; ++j) part[j] = float4_t{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
-                for (int r = 0; r < 4; ++r) part[j] = mfma_f32_16x16x4(cur.q[j][r], st[j][r], part[j]);
-            }
+        for (int r = 0; r < 4; ++r) {
+#pragma unroll
+            for (int j = 0; j < TW; ++j) part[j] = mfma_f32_16x16x4(f.q[j][r], st[j][r], part[j]);
         }
 #pragma unroll
         for (int j = 0; j < TW; ++j) {
-            if (wave * TW + j < ntiles) {
-                float4_t s = st[j];
-                mfma_results_ready<8>(s);
-                s *= cur.a[j];
+            mfma_results_ready<8>(st[j]);
+            st[j] *= f.a[j];
+        }
 #pragma unroll
-                for (int r = 0; r < 4; ++r) s = mfma_f32_16x16x4(cur.k[j][r], cur.v[r], s);
-                st[j] = s;
-            }
+        for (int r = 0; r < 4; ++r) {
+#pragma unroll
+            for (int j = 0; j < TW; ++j) st[j] = mfma_f32_16x16x4(f.k[j][r], vv[r], st[j]);
         }
         float4_t out = part[TW];
         mfma_results_ready<8>(out);
 #pragma unroll
         for (int j = 0; j < TW; ++j) {
-            float4_t p = part[j];
-            mfma_results_ready<8>(p);
-            out += p;
+            mfma_results_ready<8>(part[j]);
+            if (wave * TW + j < ntiles) out += part[j];     // (wave-uniform; a row tile beyond the state repeats the last one)
         }
         if (dskip && wave == 0) {       // (v of this lane: token 4 lq + r, column li — the layout of the result)
 #pragma unroll
-            for (int r = 0; r < 4; ++r) out[r] = fmaf(dh, cur.v[r], out[r]);
+            for (int r = 0; r < 4; ++r) out[r] = fmaf(dh, vv[r], out[r]);
         }
         float *rb = &red[i & 1][0][0];
         *reinterpret_cast<float4_t *>(rb + wave * 256 + lane * 4) = out;
@@ -222,8 +219,21 @@ __global__ __launch_bounds__(kLsThreads) void linear_scan_kernel(
         for (int w = 0; w < kLsWaves; ++w) sum += rb[w * 256 + from];
         const int tok = i * kLsTile + t;
         if (tok < cnt && col0 + c < dv) o[(row0 + tok) * o_stride + static_cast<int64_t>(h) * dv + col0 + c] = sum;
-        cur = nxt;
+    };
+    LsOperands<T, TW> f[AHEAD + 1];
+#pragma unroll
+    for (int a = 0; a < AHEAD; ++a) load(a, f[a]);
+    int i = 0;
+    for (; i + AHEAD < nt; i += AHEAD + 1) {
+#pragma unroll
+        for (int a = 0; a <= AHEAD; ++a) {
+            load(i + a + AHEAD, f[(a + AHEAD) % (AHEAD + 1)]);
+            compute(i + a, f[a]);
+        }
     }
+#pragma unroll
+    for (int a = 0; a < AHEAD; ++a)
+        if (i + a < nt) compute(i + a, f[a]);       // (uniform)
 #pragma unroll
     for (int j = 0; j < TW; ++j) {
         float4_t s = st[j];
@@ -391,7 +401,7 @@ extern "C" int swl_linear_scan(float *o, int64_t o_stride, const float *qd, cons
     const dim3 grid(static_cast<unsigned>(num_seqs), static_cast<unsigned>(num_heads), static_cast<unsigned>(shares));
 #define SWL_LS(N)                                                                                                             \
     case N:                                                                                                                   \
-        hipLaunchKernelGGL((swl::linear_scan_kernel<T, N>), grid, dim3(swl::kLsThreads), 0, static_cast<hipStream_t>(stream), o, \
+        hipLaunchKernelGGL((swl::linear_scan_kernel<T, N, (N <= 2 ? 2 : 1)>), grid, dim3(swl::kLsThreads), 0, static_cast<hipStream_t>(stream), o, \
                            o_stride, qd, kd, total, intra, static_cast<const T *>(v), v_stride, dskip, state, slot_stride, s_off, \
                            seq_row0, seq_cnt, seq_tile0, tok_pos, tok_state, num_heads, dim, dp, vdim);                       \
         break

@@ -4,7 +4,7 @@
 //     out = sigmoid(y)^p         (kind 0)      or      exp(-exp(y))     (kind 1)          fp32 [T, channels]
 // W1 [rank, width] and W2 [channels, rank] are the compute dtype, the bias, the activations and the decays fp32.
 //
-//   16-bit, width / rank / channels multiples of 16: one workgroup per (16 tokens, share of the channels) on the matrix cores. The
+//   16-bit, width a multiple of 32, rank and channels of 16: one workgroup per (16 tokens, share of the channels) on the matrix cores. The
 //   four waves share the reduction over the width (their partial z meet in LDS, where the activation is applied and z becomes a
 //   16-bit operand again), then the channel tiles.
 //   otherwise: one workgroup per token, a wave per rank row, then a thread per channel.
@@ -20,6 +20,13 @@ __device__ __forceinline__ float ld_decay(float y, int kind, float power) {
     // sigmoid(y)^p = exp(p ln sigmoid(y)), ln sigmoid(y) = min(y, 0) - ln(1 + e^-|y|)
     if (kind == 0) return expf(power * (fminf(y, 0.f) - log1pf(expf(-fabsf(y)))));
     return expf(-expf(y));
+}
+
+__device__ __forceinline__ float4_t mfma32(vec8_t<bf16> a, vec8_t<bf16> b, float4_t c) {
+    return __builtin_amdgcn_mfma_f32_16x16x32_bf16(a, b, c, 0, 0, 0);
+}
+__device__ __forceinline__ float4_t mfma32(vec8_t<f16> a, vec8_t<f16> b, float4_t c) {
+    return __builtin_amdgcn_mfma_f32_16x16x32_f16(a, b, c, 0, 0, 0);
 }
 
 template <typename T>
@@ -64,20 +71,27 @@ __global__ __launch_bounds__(kLdThreads) void low_rank_decay_mfma_kernel(float *
     const int li = lane & 15, lq = lane >> 4;
     const int64_t last = num_tokens - 1;
     if (w1) {
-        // D[token][rank row] = sum_i x[token][i] w1[rank row][i]: A lane = token li, B lane = rank row li, both at i = 4 lq ..
+        // D[token][rank row] = sum_i x[token][i] w1[rank row][i]: A lane = token li, B lane = rank row li, both at i = 8 lq ..
         float4_t acc[RT];
 #pragma unroll
         for (int j = 0; j < RT; ++j) acc[j] = float4_t{0.f, 0.f, 0.f, 0.f};
-        const T *xr = x + (t0 + li < num_tokens ? t0 + li : last) * x_stride + 4 * lq;
-        const T *wr = w1 + static_cast<int64_t>(li) * width + 4 * lq;
-#pragma unroll 4
-        for (int i = wave * 16; i < width; i += kLdWaves * 16) {
-            vec4_t<T> a, b;
-            load4(a, xr + i);
+        const T *xr = x + (t0 + li < num_tokens ? t0 + li : last) * x_stride + 8 * lq;
+        const T *wr = w1 + static_cast<int64_t>(li) * width + 8 * lq;
+        for (int i = wave * 32; i < width; i += kLdWaves * 32 * 4) {       // four steps' operands are requested together
+            vec8_t<T> a[4], b[4][RT];
 #pragma unroll
-            for (int j = 0; j < RT; ++j) {
-                load4(b, wr + static_cast<int64_t>(j) * 16 * width + i);
-                acc[j] = mfma16(a, b, acc[j]);
+            for (int u = 0; u < 4; ++u) {
+                const int iu = min(i + u * kLdWaves * 32, width - 32);
+                a[u] = load8(xr + iu);
+#pragma unroll
+                for (int j = 0; j < RT; ++j) b[u][j] = load8(wr + static_cast<int64_t>(j) * 16 * width + iu);
+            }
+#pragma unroll
+            for (int u = 0; u < 4; ++u) {
+                if (i + u * kLdWaves * 32 < width) {        // (wave-uniform)
+#pragma unroll
+                    for (int j = 0; j < RT; ++j) acc[j] = mfma32(a[u], b[u][j], acc[j]);
+                }
             }
         }
 #pragma unroll
@@ -141,7 +155,7 @@ extern "C" int swl_low_rank_decay(float *out, const void *x, int64_t x_stride, c
     const auto eight = [](const void *p) { return (reinterpret_cast<uintptr_t>(p) & 7) == 0; };
     const int rt = rank / 16;
     if (dtype != SWL_F32 && rank % 16 == 0 && (rt == 1 || rt == 2 || rt == 4 || rt == 8) && channels % 16 == 0 &&
-        (!w1 || width % 16 == 0) && x_stride % 4 == 0 && eight(x) && eight(w1) && eight(w2)) {
+        (!w1 || (width % 32 == 0 && x_stride % 8 == 0 && swl::aligned16(x) && swl::aligned16(w1))) && eight(w2)) {
         const int64_t tiles = (num_tokens + 15) / 16;
         // few tokens: the channels are shared out over workgroups (each makes the small z again)
         int shares = 1;

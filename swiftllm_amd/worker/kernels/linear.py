@@ -258,6 +258,25 @@ def _blas_linear(a: torch.Tensor, w: torch.Tensor, row_blocks=None, plateau=None
     return out
 
 
+def linear_grouped(x: torch.Tensor, w: torch.Tensor, skinny: bool = False) -> torch.Tensor:
+    """x [groups, T, in], w [groups * out, in] -> [T, groups * out]: columns g * out .. are x[g] @ w[g * out : (g + 1) * out]^T. One
+    launch for decode-sized steps on a packed weight, a product per group otherwise."""
+    groups, m, k = x.shape
+    n = w.shape[0]
+    out = torch.empty((m, n), dtype=x.dtype, device=x.device)
+    wp = _packed_of(w)
+    if skinny and wp is not None and m <= _SKINNY_MAX_M and (n // groups) % 128 == 0 and x.is_contiguous() and _skinny_ok(x[0], w):
+        need = _hip.load().swl_gemm_skinny_workspace_bytes(m, n, k)
+        ws = _workspace(x.device, need) if need else None
+        _hip.call("swl_gemm_skinny_packed_grouped", _hip.ptr(out), _hip.ptr(x), m * k, groups, _hip.ptr(wp), _hip.ptr(ws),
+                  ws.numel() * 4 if ws is not None else 0, m, n, k, k, n, _hip.dtype_code(x.dtype), _hip.stream())
+        return out
+    size = n // groups
+    for g in range(groups):
+        torch.mm(x[g], w[g * size:(g + 1) * size].t(), out=out[:, g * size:(g + 1) * size])
+    return out
+
+
 def linear_splitk(a: torch.Tensor, w: torch.Tensor, always: bool = False):
     """Like linear(a, w, skinny=True) but returns SplitKPartials when the kernel splits K (the caller
     hands them to a fused consumer); falls through to `linear` otherwise. `always`: also return the

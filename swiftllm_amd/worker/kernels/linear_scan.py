@@ -10,6 +10,10 @@ from .rms_stream import StateRef
 DECAY_SIGMOID_POWER = 0     # sigmoid(y)^power
 DECAY_EXP_EXP = 1           # exp(-exp(y))
 
+# limits of csrc/linear_scan.hip
+STEP_MAX_VDIM = 256         # a thread of the one-token kernel owns one or four columns
+TILE_MAX_DIM = 320          # key channels of a tile in LDS
+
 
 def low_rank_decay(x: torch.Tensor, w1: torch.Tensor, w2: torch.Tensor, bias: torch.Tensor, kind: int, power: float = 1.0,
                    tanh: bool = False) -> torch.Tensor:
@@ -25,13 +29,13 @@ def low_rank_decay(x: torch.Tensor, w1: torch.Tensor, w2: torch.Tensor, bias: to
     return out
 
 
-def linear_recurrence(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, decay: torch.Tensor, st: StateRef, tiles, state_off: int,
-                      num_heads: int, dim: int, vdim: int, q_scale: float = 1.0, bonus: torch.Tensor = None,
+def linear_recurrence(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, decay: torch.Tensor, st: StateRef, state_off: int, num_heads: int,
+                      dim: int, vdim: int, q_scale: float = 1.0, bonus: torch.Tensor = None,
                       k_scale: torch.Tensor = None, dskip: torch.Tensor = None, num_qk_heads: int = 0, finish=None) -> torch.Tensor:
     """Per head, on the fp32 state [heads, dim, vdim] at state_off inside each sequence's slot: S <- diag(decay) S + k v^T, o = S^T q
     (+ dskip v); with `bonus` (fp32 [heads, dim]): o = (S + diag(bonus) k v^T)^T q of the state before the update. q [T, num_qk_heads
     * dim] (times q_scale), k likewise (times k_scale[t, h], when given), v [T, num_heads * vdim] may be column slices; decay fp32
-    [T, num_heads * dim] or [T, num_heads]. tiles = (tile_row0, tile_cnt, seq_tile0) of the plan.
+    [T, num_heads * dim] or [T, num_heads]. st.tiles: the step's tiles.
     finish None: -> o fp32 [T, num_heads * vdim]. finish = (out, norm_w, gate, eps, mult): the head norm of `gated_head_rmsnorm` is
     applied too and the result goes to `out`."""
     _hip.require_gpu_tensor(q, "q")
@@ -43,7 +47,7 @@ def linear_recurrence(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, decay: 
     per_channel = decay.shape[1] == H * dim
     for t, size in ((bonus, H * dim), (k_scale, n * H), (dskip, H)):
         assert t is None or (t.dtype == torch.float32 and t.is_contiguous() and t.numel() == size)
-    row0, cnt, seq_tile0 = tiles
+    row0, cnt, seq_tile0 = st.tiles
     num_seqs, num_tiles = st.seq_row0.shape[0], row0.shape[0]
     code, stream, dev, f32 = _hip.dtype_code3(q.dtype), _hip.stream(), q.device, torch.float32
     if num_seqs == n and vdim <= STEP_MAX_VDIM:          # every portion is one token
@@ -79,6 +83,3 @@ def linear_recurrence(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, decay: 
     out, norm_w, gate, eps, mult = finish
     gated_head_rmsnorm(out, o, gate, norm_w, H, vdim, eps, mult)
     return out
-
-
-STEP_MAX_VDIM = 256         # (csrc/linear_scan.hip: a thread of the one-token kernel owns one or four columns)

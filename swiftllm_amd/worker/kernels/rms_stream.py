@@ -55,10 +55,12 @@ def post_norm_add(x: torch.Tensor, a: torch.Tensor, post: torch.Tensor, b: torch
 
 
 class StateRef:
-    """Where a step's kernels find per-sequence state: the slot pool, and the plan's per-token arrays."""
-    __slots__ = ("pool", "tok_pos", "tok_start", "tok_state", "tok_seq", "seq_row0", "seq_cnt")
+    """Where a step's kernels find per-sequence state: the slot pool, and the plan's per-token arrays. tiles (tile_row0, tile_cnt,
+    seq_tile0): the portions cut into runs of up to 16 tokens, for recurrences that run by tiles."""
+    __slots__ = ("pool", "tok_pos", "tok_start", "tok_state", "tok_seq", "seq_row0", "seq_cnt", "tiles")
 
-    def __init__(self, pool, tok_pos, tok_start, tok_state, tok_seq, seq_row0, seq_cnt):
+    def __init__(self, pool, tok_pos, tok_start, tok_state, tok_seq, seq_row0, seq_cnt, tiles=None):
+        self.tiles = tiles
         self.pool, self.tok_pos, self.tok_start, self.tok_state = pool, tok_pos, tok_start, tok_state
         self.tok_seq, self.seq_row0, self.seq_cnt = tok_seq, seq_row0, seq_cnt
 

@@ -4,7 +4,7 @@ import torch
 
 from swiftllm_amd import _hip
 
-from ..kernels.linear import linear, linear_silu_gate
+from ..kernels.linear import linear, linear_silu_gate, linear_splitk
 from ..kernels.moe import ACT_SILU_UP_FIRST, gated_unit, moe_experts, moe_route
 from ..kernels.polynorm import polynorm
 from ..kernels.window_attn import qknorm_and_store_kv, window_attention
@@ -25,6 +25,18 @@ def _project(a: torch.Tensor, w: torch.Tensor, skinny: bool) -> torch.Tensor:
                 raise
             w._swl_blas_only = True
     return linear(a, w, False)
+
+
+def _project_partials(a: torch.Tensor, w: torch.Tensor, skinny: bool):
+    """_project for a consumer that takes a product's K shares too: SplitKPartials where the decode GEMM splits K, rows otherwise."""
+    if skinny and a.dtype != torch.float32 and not getattr(w, "_swl_blas_only", False):
+        try:
+            return linear_splitk(a, w)
+        except _hip.HipLibraryError as exc:
+            if "code -2" not in str(exc):       # (see _project)
+                raise
+            w._swl_blas_only = True
+    return _project(a, w, skinny)
 
 
 def _silu_unit(a: torch.Tensor, up_gate: torch.Tensor, skinny: bool) -> torch.Tensor:

@@ -11,13 +11,12 @@ from swiftllm_amd import _hip
 
 class StepContext:
     """What the sublayers of one step share: the block pool and table, the per-token plan arrays, the state slots, the portions'
-    chunks (chunk_row0, chunk_cnt, seq_chunk0: designs whose recurrence runs in parallel over them), the portions' first tiles."""
-    __slots__ = ("pool", "block_table", "tok_seq", "tok_pos", "tiles", "state", "chunks", "seq_tile0")
+    chunks (chunk_row0, chunk_cnt, seq_chunk0: designs whose recurrence runs in parallel over them)."""
+    __slots__ = ("pool", "block_table", "tok_seq", "tok_pos", "tiles", "state", "chunks")
 
-    def __init__(self, pool, block_table, tok_seq, tok_pos, tiles, state, chunks=None, seq_tile0=None):
+    def __init__(self, pool, block_table, tok_seq, tok_pos, tiles, state, chunks=None):
         self.pool, self.block_table, self.tok_seq, self.tok_pos, self.tiles, self.state, self.chunks = \
             pool, block_table, tok_seq, tok_pos, tiles, state, chunks
-        self.seq_tile0 = seq_tile0
 
 
 class LorulixAttention:

@@ -4,12 +4,13 @@ next input's norm are the model's fused step (kernels/hyper_stream.py)."""
 import torch
 
 from ..kernels.linear_scan import DECAY_EXP_EXP, DECAY_SIGMOID_POWER, linear_recurrence, low_rank_decay
+from ..kernels.linear import linear_grouped
 from ..kernels.moe import gated_rows
 from ..kernels.rms_stream import token_shift_mix
 from ..kernels.rope_kv import qkv_conv_rope_and_store_kv
 from ..kernels.ssd import state_space_mixer
 from ..kernels.window_attn import MASK_CHUNK, MASK_WINDOW, AttentionSpec, masked_attention
-from .kekapel_layer import _project
+from .kekapel_layer import _project, _project_partials
 from .lorulix_layer import StepContext
 
 
@@ -51,7 +52,7 @@ class _LinearAttention:
         mx, w = self.mixer, self.w
         decay = low_rank_decay(proj[:, w.cols["decay"]], None, w.decay_2, w.decay_b, DECAY_SIGMOID_POWER, 1.0 / mx.tau)
         q, k, v, g = (proj[:, w.cols["right_" + n]] for n in "qkvg")
-        linear_recurrence(q, k, v, decay, ctx.state, ctx.tiles + (ctx.seq_tile0,), self.state_off, mx.num_heads, mx.key_dim,
+        linear_recurrence(q, k, v, decay, ctx.state, self.state_off, mx.num_heads, mx.key_dim,
                           mx.value_dim, q_scale=mx.key_dim ** -0.5,
                           finish=(row[:, w.ins["right"]], w.right_norm, g, self.eps, self.mult))
 
@@ -67,9 +68,10 @@ class _TimeMixing:
     def forward(self, h: torch.Tensor, proj: torch.Tensor, row: torch.Tensor, ctx: StepContext, skinny: bool):
         mx, w = self.mixer, self.w
         mixes = token_shift_mix(h, w.mu, ctx.state, self.tail_off)
-        r, k, v, g = (_project(mixes[i], m, skinny) for i, m in enumerate(w.shifted))
+        rkvg = linear_grouped(mixes[:4], w.shifted, skinny)
+        r, k, v, g = (rkvg[:, i * mx.inner:(i + 1) * mx.inner] for i in range(4))
         decay = low_rank_decay(mixes[4], w.decay_1, w.decay_2, w.decay_b, DECAY_EXP_EXP, tanh=True)
-        linear_recurrence(r, k, v, decay, ctx.state, ctx.tiles + (ctx.seq_tile0,), self.state_off, mx.num_heads, mx.key_dim,
+        linear_recurrence(r, k, v, decay, ctx.state, self.state_off, mx.num_heads, mx.key_dim,
                           mx.value_dim, bonus=w.bonus, finish=(row[:, w.ins["right"]], w.right_norm, g, self.eps, self.mult))
 
 
@@ -102,7 +104,8 @@ class VafozenLayer:
             shift = state.add_region(2 * weight.mu.shape[1])
             self.right = _TimeMixing(layer_config, weight, eps, shift, state.add_region(rt.state_elems))
 
-    def forward(self, h: torch.Tensor, ctx: StepContext) -> torch.Tensor:
+    def forward(self, h: torch.Tensor, ctx: StepContext):
+        """-> the layer's result, rows or SplitKPartials."""
         w = self.w
         proj = _project(h, w.proj, self.skinny)
         make = torch.zeros if w.row_gaps else torch.empty       # (columns of no piece meet zero weights: they must be finite)
@@ -112,4 +115,4 @@ class VafozenLayer:
         self.right.forward(h, proj, row, ctx, self.skinny)
         if self.mlp is not None:
             gated_rows(row[:, w.ins["ff"]], proj[:, w.cols["ff_gate"]], proj[:, w.cols["ff_up"]])
-        return _project(row, w.out, self.skinny)
+        return _project_partials(row, w.out, self.skinny)

@@ -84,9 +84,9 @@ class VafozenModel(SteppedModel):
         cfg, w = self.model_config, self.weight
         eps, plain = cfg.norm_eps, self._plain
         st = StateRef(self.state.pool, dev["tok_pos"], dev["tok_start"], dev["tok_state"], dev["tok_seq"], dev["seq_row0"],
-                      dev["seq_cnt"])
+                      dev["seq_cnt"], (dev["tile_row0"], dev["tile_cnt"], dev["seq_tile0"]))
         ctx = StepContext(self.kv_pool if use_pool else None, self.gpu_block_manager.block_table if use_pool else None,
-                          dev["tok_seq"], dev["tok_pos"], (dev["tile_row0"], dev["tile_cnt"]), st, seq_tile0=dev["seq_tile0"])
+                          dev["tok_seq"], dev["tok_pos"], (dev["tile_row0"], dev["tile_cnt"]), st)
         x, _ = embed_positions(dev["input_ids"], dev["tok_pos"], w.embed, None, cfg.embedding_scale, keep_copy=False)
         x = x.unsqueeze(1)
         tap, layers = self.layer_tap, w.layers

@@ -9,7 +9,8 @@ way in and ONE on the way out:
     pieces on multiples of 8 rows (16-byte boundaries in the product), zero rows between;
   * `out`: the output projections side by side along the input dimension (`ins[name]` likewise). What precedes it writes into one
     row per token; the factors of the two mixers are applied there (left: to the values as they are cached, right: by the head norm).
-Time mixing reads token-shifted mixes of the input, so its r / k / v / gate matrices stay on their own ([4, inner, width]).
+Time mixing reads token-shifted mixes of the input, so its r / k / v / gate matrices are a stack of their own (`shifted`, [4 inner, width]:
+one grouped product).
 Low-rank decay matrices are padded with zero rows / columns to a rank that is a power of two from 16 on (what the matrix-core form
 takes) in 16-bit models; their rank is the checkpoint tensor's.
 Everything that enters fp32 arithmetic — norm weights (the layers' and the model's are stored around zero: kept as 1 + w), biases, q/k
@@ -121,7 +122,7 @@ class VafozenLayerWeight:
                     self.conv = torch.cat([f32(f"{q}{n}.conv", (s, lf.conv_taps)) for n, s in sizes.items()]).t().contiguous()
                 ins.add("gate", mat(q + "g", (lf.o_size, w)))
                 self.mu = torch.stack([f32(f"{r}mu.{s}", (w,)) for s in "rkvgw"]).contiguous()
-                self.shifted = [mat(r + s, (rt.inner, w)) for s in "rkvg"]
+                self.shifted = torch.cat([mat(r + s, (rt.inner, w)) for s in "rkvg"]).contiguous()
                 self.decay_1, self.decay_2 = low_rank(r + "w1", r + "w2", rt.keys)
                 self.decay_b = f32(r + "w0", (rt.keys,))
                 self.bonus = f32(r + "u", (rt.num_heads, rt.key_dim))
@@ -155,7 +156,7 @@ class VafozenWeight:
         """The 2-D matrices a step multiplies through `linear` (candidates for the decode GEMMs' packed copies)."""
         out = [self.head]
         for layer in self.layers:
-            out += [layer.proj, layer.out] + getattr(layer, "shifted", [])
+            out += [layer.proj, layer.out] + ([layer.shifted] if hasattr(layer, "shifted") else [])
         return out
 
 
