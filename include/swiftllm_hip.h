@@ -31,7 +31,8 @@
 extern "C" {
 #endif
 
-#define SWL_ABI_VERSION 1
+/* raised whenever the parameters of an existing entry point change */
+#define SWL_ABI_VERSION 2
 
 #define SWL_F16 0
 #define SWL_BF16 1

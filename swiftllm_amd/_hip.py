@@ -21,7 +21,7 @@ _LIB_PATH = os.path.join(os.path.dirname(os.path.abspath(__file__)), "csrc", _LI
 SWL_F16 = 0
 SWL_BF16 = 1
 SWL_F32 = 2     # only the operators that say so accept it
-ABI_VERSION = 1
+ABI_VERSION = 2
 
 _P = ctypes.c_void_p
 _I32 = ctypes.c_int32

@@ -8,8 +8,10 @@ and travels to the GPU box with the repo snapshot.
 import argparse
 import concurrent.futures
 import os
+import re
 import shutil
 import subprocess
+import sys
 import tempfile
 
 HERE = os.path.dirname(os.path.abspath(__file__))
@@ -72,6 +74,28 @@ CXXFLAGS = [f"--offload-arch={ARCH}", "-O3", "-std=c++17", "-fPIC", "-ffp-contra
             "-Wno-unused-function",
             # the compiler may not form packed-fp32 VALU ops from scalar float code
             "-Xclang", "-target-feature", "-Xclang", "-packed-fp32-ops"]
+
+
+def entry_points(sources):
+    """The C entry points that the given sources define."""
+    out = []
+    for src in sources:
+        with open(os.path.join(HERE, src), "r", encoding="utf-8") as f:
+            out += re.findall(r'^extern "C" [^(]*?\b(swl_\w+)\(', f.read(), flags=re.M)
+    return out
+
+
+def serves(sources, lib: str = LIB) -> bool:
+    """Whether the built library has this tree's ABI version and every entry point of `sources` (a library built for one model family
+    lacks the others'; one built before an interface changed has another version). Asked in a child process: a library that is loaded
+    here could not be replaced any more."""
+    if not os.path.exists(lib):
+        return False
+    with open(os.path.join(ROOT, "include", "swiftllm_hip.h"), "r", encoding="utf-8") as f:
+        version = re.search(r"#define SWL_ABI_VERSION (\d+)", f.read()).group(1)
+    ask = ("import ctypes, sys; lib = ctypes.CDLL(sys.argv[1]); "
+           "sys.exit(0 if lib.swl_abi_version() == int(sys.argv[2]) and all(hasattr(lib, n) for n in sys.argv[3:]) else 3)")
+    return subprocess.run([sys.executable, "-c", ask, lib, version, *entry_points(sources)], capture_output=True).returncode != 3
 
 
 def _hipcc() -> str:
