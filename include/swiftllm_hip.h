@@ -714,7 +714,8 @@ int swl_delta_rule(float *o, const float *qn, const float *kn, const float *kq, 
                    const int32_t *tok_pos, const int32_t *tok_state, int32_t num_seqs, int32_t num_heads,
                    int32_t num_qk_heads, int32_t dim, int32_t vdim, swl_stream_t stream);
 int swl_gated_head_rmsnorm(void *out, int64_t out_stride, const float *o, const void *gate, int64_t gate_stride, const float *w,
-                           int32_t w_head_stride, float mult, float eps, int64_t num_tokens, int32_t num_heads, int32_t vdim, int32_t dtype, swl_stream_t stream);
+                           int32_t w_head_stride, float mult, float eps, int64_t num_tokens, int32_t num_heads, int32_t vdim,
+                           int32_t dtype, swl_stream_t stream);
 
 /* ---- sigmoid router with group-limited choice (csrc/moe.hip) ---------------------------------------------------------------
  * s = sigmoid(router[experts, width] h) in fp32. Experts are chosen by s + correction (NULL: by s): the experts form
@@ -772,7 +773,8 @@ int swl_ssd_scan(float *y, const float *xbc, const float *dt, const float *decay
                  int64_t slot_stride, int64_t s_off, const int32_t *seq_row0, const int32_t *seq_cnt, const int32_t *tok_pos,
                  const int32_t *tok_state, int32_t num_seqs, int32_t num_heads, int32_t vdim, int32_t state_dim,
                  int32_t groups, swl_stream_t stream);
-int swl_gated_group_rmsnorm(void *out, int64_t out_stride, const float *y, const void *gate, int64_t gate_stride, const float *w, float eps,
+int swl_gated_group_rmsnorm(void *out, int64_t out_stride, const float *y, const void *gate, int64_t gate_stride, const float *w,
+                            float eps,
                             int64_t num_tokens, int32_t cols, int32_t groups, int32_t dtype, swl_stream_t stream);
 
 /* ---- fp32 stream of models that norm a sublayer's RESULT only (csrc/rms_stream.hip) -----------------------------------------
@@ -844,13 +846,15 @@ int swl_low_rank_decay(float *out, const void *x, int64_t x_stride, const void *
 /* ---- fp32 residual of several streams, hyper-connections (csrc/hyper_stream.hip) ------------------------------------------------
  * x [rows, streams, width] fp32. swl_embed_streams: every stream = embed[token]. swl_hyper_step: with y (+ y2, + y_bias[width])
  * the previous sublayer's result (the fp32 sum of y_parts rows y[t * y_parts + j], or — y NULL, slabs given — of the y_parts fp32
- * slabs [rows, width] that lie slab_stride elements apart: a product's K shares), X_t <- sum_s mix[s][t] X_s + outw[t] y (all from the old streams); then, with h given,
+ * slabs [rows, width] that lie slab_stride elements apart: a product's K shares), X_t <- sum_s mix[s][t] X_s + outw[t] y (all from
+ * the old streams); then, with h given,
  * u = sum_s inw[s] X_s (inw NULL: plain sum) and h = u / rms(u in `groups` equal parts; eps) * norm_w. y NULL: norm only, of
  * rows row_idx when given; h NULL: update only. At most 16 streams. dtype (y, y2, h) may be SWL_F32. */
 int swl_embed_streams(float *x, const void *embed, const int32_t *tokens, int64_t num_tokens, int32_t width, int32_t streams,
                       int32_t dtype, swl_stream_t stream);
 int swl_hyper_step(float *x, const void *y, int32_t y_parts, const float *slabs, int64_t slab_stride, const void *y2,
-                   const float *y_bias, const float *mix, const float *outw, const float *inw, const float *norm_w, void *h, const int32_t *row_idx, int64_t num_rows,
+                   const float *y_bias, const float *mix, const float *outw, const float *inw, const float *norm_w, void *h,
+                   const int32_t *row_idx, int64_t num_rows,
                    int32_t width, int32_t streams, int32_t groups, float eps, int32_t dtype, swl_stream_t stream);
 
 /* ---- minGRU (csrc/min_gru.hip) -----------------------------------------------------------------------------------------------------

@@ -361,7 +361,8 @@ extern "C" int swl_delta_rule(float *o, const float *qn, const float *kn, const 
 }
 
 extern "C" int swl_gated_head_rmsnorm(void *out, int64_t out_stride, const float *o, const void *gate, int64_t gate_stride,
-                                      const float *w, int32_t w_head_stride, float mult, float eps, int64_t num_tokens, int32_t num_heads, int32_t vdim, int32_t dtype,
+                                      const float *w, int32_t w_head_stride, float mult, float eps, int64_t num_tokens,
+                                      int32_t num_heads, int32_t vdim, int32_t dtype,
                                       swl_stream_t stream) {
     if (num_tokens < 0 || num_heads <= 0 || vdim <= 0 || gate_stride < static_cast<int64_t>(num_heads) * vdim ||
         out_stride < static_cast<int64_t>(num_heads) * vdim)

@@ -214,7 +214,8 @@ inline size_t hs_lds_bytes(int width, int groups) {
 }
 
 template <typename T, int V>
-void launch_hs(dim3 grid, size_t lds, hipStream_t s, float *x, const T *y, int yp, const float *sl, int64_t ss, const T *y2, const float *yb, const float *mix,
+void launch_hs(dim3 grid, size_t lds, hipStream_t s, float *x, const T *y, int yp, const float *sl, int64_t ss, const T *y2,
+               const float *yb, const float *mix,
                const float *ow, const float *iw, const float *nw, T *h, const int32_t *ri, int width, int streams, int groups,
                float eps) {
 #define SWL_HS(S, X)                                                                                                          \
@@ -249,7 +250,8 @@ extern "C" int swl_embed_streams(float *x, const void *embed, const int32_t *tok
 }
 
 extern "C" int swl_hyper_step(float *x, const void *y, int32_t y_parts, const float *slabs, int64_t slab_stride, const void *y2,
-                              const float *y_bias, const float *mix, const float *outw, const float *inw, const float *norm_w, void *h, const int32_t *row_idx,
+                              const float *y_bias, const float *mix, const float *outw, const float *inw, const float *norm_w, void *h,
+                              const int32_t *row_idx,
                               int64_t num_rows, int32_t width, int32_t streams, int32_t groups, float eps, int32_t dtype,
                               swl_stream_t stream) {
     const bool has_y = y || slabs;
@@ -268,10 +270,12 @@ extern "C" int swl_hyper_step(float *x, const void *y, int32_t y_parts, const fl
     hipStream_t s = static_cast<hipStream_t>(stream);
     SWL_DISPATCH_DTYPE3(dtype, T, {
         if (wide)
-            swl::launch_hs<T, 4>(grid, lds, s, x, static_cast<const T *>(y), y_parts, slabs, slab_stride, static_cast<const T *>(y2), y_bias, mix, outw, inw,
+            swl::launch_hs<T, 4>(grid, lds, s, x, static_cast<const T *>(y), y_parts, slabs, slab_stride, static_cast<const T *>(y2),
+                                 y_bias, mix, outw, inw,
                                  norm_w, static_cast<T *>(h), row_idx, width, streams, groups, eps);
         else
-            swl::launch_hs<T, 1>(grid, lds, s, x, static_cast<const T *>(y), y_parts, slabs, slab_stride, static_cast<const T *>(y2), y_bias, mix, outw, inw,
+            swl::launch_hs<T, 1>(grid, lds, s, x, static_cast<const T *>(y), y_parts, slabs, slab_stride, static_cast<const T *>(y2),
+                                 y_bias, mix, outw, inw,
                                  norm_w, static_cast<T *>(h), row_idx, width, streams, groups, eps);
     });
     return swl::check_launch();

@@ -401,8 +401,9 @@ extern "C" int swl_linear_scan(float *o, int64_t o_stride, const float *qd, cons
     const dim3 grid(static_cast<unsigned>(num_seqs), static_cast<unsigned>(num_heads), static_cast<unsigned>(shares));
 #define SWL_LS(N)                                                                                                             \
     case N:                                                                                                                   \
-        hipLaunchKernelGGL((swl::linear_scan_kernel<T, N, (N <= 2 ? 2 : 1)>), grid, dim3(swl::kLsThreads), 0, static_cast<hipStream_t>(stream), o, \
-                           o_stride, qd, kd, total, intra, static_cast<const T *>(v), v_stride, dskip, state, slot_stride, s_off, \
+        hipLaunchKernelGGL((swl::linear_scan_kernel<T, N, (N <= 2 ? 2 : 1)>), grid, dim3(swl::kLsThreads), 0,                 \
+                           static_cast<hipStream_t>(stream), o, o_stride, qd, kd, total, intra,                         \
+                           static_cast<const T *>(v), v_stride, dskip, state, slot_stride, s_off,                             \
                            seq_row0, seq_cnt, seq_tile0, tok_pos, tok_state, num_heads, dim, dp, vdim);                       \
         break
     SWL_DISPATCH_DTYPE3(dtype, T, {

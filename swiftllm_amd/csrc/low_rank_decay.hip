@@ -4,8 +4,8 @@
 //     out = sigmoid(y)^p         (kind 0)      or      exp(-exp(y))     (kind 1)          fp32 [T, channels]
 // W1 [rank, width] and W2 [channels, rank] are the compute dtype, the bias, the activations and the decays fp32.
 //
-//   16-bit, width a multiple of 32, rank and channels of 16: one workgroup per (16 tokens, share of the channels) on the matrix cores. The
-//   waves share the reduction over the width (their partial z meet in LDS, where the activation is applied and z becomes a
+//   16-bit, width a multiple of 32, rank and channels of 16: one workgroup per (16 tokens, share of the channels) on the matrix
+//   cores. The waves share the reduction over the width (their partial z meet in LDS, where the activation is applied and z becomes a
 //   16-bit operand again), then the channel tiles, a tile's weights requested while the one before is computed.
 //   otherwise: one workgroup per token, a wave per rank row, then a thread per channel.
 #include "swl_common.h"
@@ -181,7 +181,8 @@ extern "C" int swl_low_rank_decay(float *out, const void *x, int64_t x_stride, c
         const dim3 grid(static_cast<unsigned>(tiles), static_cast<unsigned>(shares));
 #define SWL_LD(N)                                                                                                             \
     case N:                                                                                                                   \
-        hipLaunchKernelGGL((swl::low_rank_decay_mfma_kernel<T, N, (N <= 4 ? 8 : 4)>), grid, dim3(waves * 64), 0, s, out, static_cast<const T *>(x), \
+        hipLaunchKernelGGL((swl::low_rank_decay_mfma_kernel<T, N, (N <= 4 ? 8 : 4)>), grid, dim3(waves * 64), 0, s, out,       \
+                           static_cast<const T *>(x),                                                                        \
                            x_stride, static_cast<const T *>(w1), static_cast<const T *>(w2), bias, num_tokens, width, channels, act, \
                            kind, power);                                                                                      \
         break

@@ -15,7 +15,8 @@
 // The general entry point (swl_masked_attn_tiles) adds: mask_kind 1 (chunked visibility: keys [floor(p / window) * window, p]),
 // sink[H] (a logit per head that joins the denominator only), num_v_heads (value head = key head % num_v_heads: score maps
 // that share their values), out_f32 (fp32 result), slopes[H] (slope x distance off the capped score), out_dim / out_stride / gate (the
-// first out_dim of the DV value columns, into a column slice of wider rows, times the sigmoid of a gate element), and a split of the heads over blockIdx.z (head_groups: every group of
+// first out_dim of the DV value columns, into a column slice of wider rows, times the sigmoid of a gate element), and a split of the
+// heads over blockIdx.z (head_groups: every group of
 // heads_per_group heads is a workgroup of its own — many heads over one shared key head, wide value heads).
 //
 // HEADS mode (decode steps of a layer whose heads all read ONE key head, e.g. latent attention): a tile is one token and the
@@ -518,7 +519,8 @@ extern "C" int swl_masked_attn_tiles(void *out, const void *q, const void *k_cac
                                           static_cast<const T *>(k_cache), static_cast<const T *>(v_cache), block_table, \
                                           tok_seq, tok_pos, tile_row0, tile_cnt, talk, rel, rel_len, num_q_heads, num_kv_heads, \
                                           q_tok_stride, window, scale, softcap, max_blocks_per_seq, block_stride, part_o, \
-                                          part_ml, num_tokens, nbuf, mask_kind, sink, num_v_heads, out_f32, hpg, heads_mode, slopes, out_dim, out_stride, \
+                                          part_ml, num_tokens, nbuf, mask_kind, sink, num_v_heads, out_f32, hpg, heads_mode, slopes, \
+                                          out_dim, out_stride,                                                                \
                                           static_cast<const T *>(gate), gate_stride);
 #define SWL_WM_SHAPE_MIX(DD, DDV) SWL_WM_SHAPE_(DD, DDV, true)
 #define SWL_WM_SHAPE_PLAIN(DD, DDV) SWL_WM_SHAPE_(DD, DDV, false)

@@ -39,7 +39,8 @@ def hyper_step(x: torch.Tensor, y: torch.Tensor = None, done: StreamWeights = No
                eps: float = 1e-6, out_dtype: torch.dtype = None, row_idx: torch.Tensor = None) -> torch.Tensor:
     """The step between two sublayers on the streams x [T, S, width], in place. y (+ y2, + y_bias [width] fp32): the result of the
     sublayer whose StreamWeights are `done`; y has one row per token, or k neighbouring ones (the results of its k experts) that
-    are summed, or is a product's SplitKPartials, whose fp32 slabs are summed. norm (fp32 [width]): returns the next input, the sum of the streams weighted by
+    are summed, or is a product's SplitKPartials, whose fp32 slabs are summed. norm (fp32 [width]): returns the next input, the sum of
+    the streams weighted by
     `read` (None: plainly summed), RMS-normed in `groups` equal parts and scaled by `norm`, in y's dtype (out_dtype without a y) —
     of rows row_idx only, when given; then y must be None."""
     _hip.require_gpu_tensor(x, "x")

@@ -29,8 +29,8 @@ def low_rank_decay(x: torch.Tensor, w1: torch.Tensor, w2: torch.Tensor, bias: to
     return out
 
 
-def linear_recurrence(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, decay: torch.Tensor, st: StateRef, state_off: int, num_heads: int,
-                      dim: int, vdim: int, q_scale: float = 1.0, bonus: torch.Tensor = None,
+def linear_recurrence(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, decay: torch.Tensor, st: StateRef, state_off: int,
+                      num_heads: int, dim: int, vdim: int, q_scale: float = 1.0, bonus: torch.Tensor = None,
                       k_scale: torch.Tensor = None, dskip: torch.Tensor = None, num_qk_heads: int = 0, finish=None) -> torch.Tensor:
     """Per head, on the fp32 state [heads, dim, vdim] at state_off inside each sequence's slot: S <- diag(decay) S + k v^T, o = S^T q
     (+ dskip v); with `bonus` (fp32 [heads, dim]): o = (S + diag(bonus) k v^T)^T q of the state before the update. q [T, num_qk_heads

@@ -179,7 +179,8 @@ class AttentionSpec:
     """Shape and constants of one attention over the pool, as the kernels see it (which need not be how the design counts
     its heads: two score maps over shared values are 2 H query heads, 2 G key heads and G value heads).
     num_v_heads: value heads in a page; key head g reads value head g % num_v_heads. slopes: fp32 [num_q_heads], slope times the
-    distance query - key is taken off the score, or None. out_dim: value columns that count (the pages' rows may be wider). window: sliding window or chunk size
+    distance query - key is taken off the score, or None. out_dim: value columns that count (the pages' rows may be wider). window:
+    sliding window or chunk size
     (mask_kind), 0 for every earlier key. sink: fp32 [num_q_heads] logits that join the denominators, or None."""
     __slots__ = ("num_q_heads", "num_kv_heads", "num_v_heads", "head_dim", "value_dim", "window", "mask_kind", "scale",
                  "softcap", "sink", "out_f32", "slopes", "out_dim")

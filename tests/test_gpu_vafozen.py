@@ -588,7 +588,8 @@ def test_keys_just_inside_and_just_outside_the_chunk(tiled, dtype, chunk):
     for other_chunk in (chunk + 1, chunk - 1, 0):
         if chunk == 1 and other_chunk == 0:
             continue
-        wrong = dict(layer, mixer=dict(layer["mixer"], left=dict(layer["mixer"]["left"], mask={"size": other_chunk} if other_chunk else None)))
+        left = dict(layer["mixer"]["left"], mask={"size": other_chunk} if other_chunk else None)
+        wrong = dict(layer, mixer=dict(layer["mixer"], left=left))
         assert (oracle_layer(wrong, W, h) - want).abs().max() > 3 * layer_tol(dtype, want), other_chunk
 
 

@@ -5,7 +5,7 @@ swiftllm_amd: the tests compare the framework's kernels, cache and state handlin
 Notation: h [T, width] is the one normed input that both halves of a layer read, W["name"] a checkpoint tensor, positions i
 (query) and j (key) count from 0, S a recurrent state of one head [key channels, value channels].
 
-    layer:       x <- x + mixer(h) + ff(h),   h = N(x) = x / sqrt(mean(x^2) + eps) * (1 + w)
+    layer:       x <- x + mixer(h) + ff(h),   h = N(x) = (1 + w) x / r(x),  r(x)^2 = mean(x^2) + eps
     parallel:    a softmax attention (biases, weighted q/k norm, scale q.k - slope_h (i - j), keys of the query's own chunk)
                  and a linear attention with a decay per key channel: S <- diag(alpha) S + k v^T, o = S^T q
     parallel_2:  a softmax attention (biases, causal convolutions, rotation by halves, capped scores, element-wise gate)
@@ -32,7 +32,7 @@ def silu(z: torch.Tensor) -> torch.Tensor:
 
 
 def causal_conv(u: torch.Tensor, w: torch.Tensor) -> torch.Tensor:
-    """u [T, C], w [C, taps]: y_t = sum_j w[:, j] u_(t - taps + 1 + j), zeros before the start."""
+    """u [T, C], w [C, taps]: y_t = sum over lags l of w[:, taps - 1 - l] u_(t - l), where u is zero at negative times."""
     T, C = u.shape
     taps = w.shape[1]
     padded = torch.cat((torch.zeros(taps - 1, C, dtype=u.dtype), u), dim=0)
